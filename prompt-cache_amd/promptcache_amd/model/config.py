@@ -855,6 +855,171 @@ class BepepelShape:
         return cls(vocab_size=vocab, hidden_size=width, norm_eps=1e-6, layers=layers, residual_mult=0.5, logit_scale=1.0, name=name)
 
 
+@dataclass
+class PikadraLayer:
+    """One layer of a Pikadra stack: latent attention (``heads`` heads of ``dim`` unrotated + ``rot_dim`` rotated query / key columns
+    and ``vdim`` value columns; queries through a latent of ``q_rank`` columns, keys and values through one of ``kv_rank`` that is
+    what a token leaves in the cache, next to ONE rotated key part for all heads) and, beside it on the same input, a feed-forward.
+
+    ``ff_kind``: "" (none), "dense" (a gated SiLU unit of width ``ff``) or "moe" (``experts`` gated SiLU units of width ``expert_ff``
+    of which each token uses the ``top`` with the largest softmax scores, weighted by those scores as they are, plus --
+    ``shared_ff`` > 0 -- one unit of that width for every token, times a sigmoid of the token's own)."""
+    heads: int
+    dim: int
+    rot_dim: int
+    vdim: int
+    kv_rank: int
+    q_rank: int
+    scale: float
+    rot_base: float = 10000.0
+    rot_dims: int = 0
+    ff_kind: str = ""
+    ff: int = 0
+    experts: int = 0
+    top: int = 0
+    expert_ff: int = 0
+    shared_ff: int = 0
+
+    kind = "latent_attention"
+
+
+@dataclass
+class PikadraShape:
+    """Pikadra: decoder-only, parallel layers (one RMS norm, whose gain is stored around zero, feeds a latent attention and a dense
+    or mixture-of-experts feed-forward; both results join the residual together), a run of layers that repeats ``loop_times`` times
+    with the same weights -- each pass with a cache of its own, entered through a projection of [stream; embedding output] plus a
+    vector of the pass --, tied embeddings scaled on the way in, logits scaled and soft-capped.  Every size and constant comes
+    from ``config.json`` (``from_config``); ``loop_times`` 0: no layer repeats; ``logit_softcap`` 0: no cap."""
+    vocab_size: int
+    hidden_size: int
+    norm_eps: float
+    layers: list
+    embed_scale: float = 1.0
+    loop_start: int = 0
+    loop_stop: int = 0
+    loop_times: int = 0
+    logit_scale: float = 1.0
+    logit_softcap: float = 0.0
+    name: str = "pikadra"
+
+    ARCHITECTURE = "Pikadra"
+    KINDS = ("latent_attention",)
+
+    @property
+    def num_hidden_layers(self) -> int:
+        return len(self.layers)
+
+    def runs(self) -> list:
+        """The layer runs of one forward in order: (layer, pass that starts right before this run or -1)."""
+        if not self.loop_times:
+            return [(i, -1) for i in range(len(self.layers))]
+        out = [(i, -1) for i in range(self.loop_start)]
+        for t in range(self.loop_times):
+            out += [(i, t if i == self.loop_start else -1) for i in range(self.loop_start, self.loop_stop)]
+        return out + [(i, -1) for i in range(self.loop_stop, len(self.layers))]
+
+    @classmethod
+    def from_config(cls, c: dict, name: str = "pikadra") -> "PikadraShape":
+        if c.get("architecture") != cls.ARCHITECTURE:
+            raise ValueError(f"config.json describes {c.get('architecture')!r}, not {cls.ARCHITECTURE}")
+        layers = []
+        for i, lc in enumerate(c["layers"]):
+            kind, m = lc.get("type"), lc.get("mixer") or {}
+            if kind not in cls.KINDS:
+                raise ValueError(f"layer {i}: unknown mixer type {kind!r}")
+            dim, rot_dim, rot = int(m["dim"]), int(m.get("rot_dim") or 0), m.get("rot") or {}
+            lay = PikadraLayer(heads=int(m["heads"]), dim=dim, rot_dim=rot_dim, vdim=int(m.get("vdim") or dim), kv_rank=int(m["kv_rank"]),
+                               q_rank=int(m["q_rank"]), scale=float(m.get("scale", (dim + rot_dim) ** -0.5)),
+                               rot_base=float(rot.get("base", 10000.0)), rot_dims=int(rot.get("dims", rot_dim)) if rot else 0)
+            mlp = lc.get("mlp")
+            if mlp:
+                fk = mlp.get("kind", "dense")
+                if fk == "dense":
+                    lay.ff_kind, lay.ff = "dense", int(mlp["ff"])
+                elif fk == "moe":
+                    lay.ff_kind, lay.experts, lay.top = "moe", int(mlp["router"]["experts"]), int(mlp["router"]["top"])
+                    lay.expert_ff = int(mlp["expert"]["ff"])
+                    lay.shared_ff = int((mlp.get("shared") or {}).get("ff") or 0)
+                else:
+                    raise ValueError(f"layer {i}: unknown feed-forward kind {fk!r}")
+            layers.append(lay)
+        loop = c.get("loop") or {}
+        shape = cls(vocab_size=int(c["vocab"]), hidden_size=int(c["width"]), norm_eps=float((c.get("norm") or {}).get("eps", 1e-6)),
+                    layers=layers, embed_scale=float((c.get("embedding") or {}).get("scale", 1.0)),
+                    loop_start=int(loop.get("start", 0)), loop_stop=int(loop.get("stop", len(layers))) if loop else 0,
+                    loop_times=int(loop.get("times", 1)) if loop else 0,
+                    logit_scale=float(c.get("logit_scale", 1.0)), logit_softcap=float(c.get("logit_softcap") or 0.0), name=name)
+        shape.check()
+        return shape
+
+    def check(self) -> None:
+        for i, l in enumerate(self.layers):
+            if min(l.heads, l.dim, l.vdim, l.kv_rank, l.q_rank) < 1 or l.rot_dim < 0:
+                raise ValueError(f"layer {i}: latent attention needs heads, head sizes and both ranks")
+            if l.rot_dims % 2 or l.rot_dims > l.rot_dim:
+                raise ValueError(f"layer {i}: {l.rot_dims} rotated columns of a part of {l.rot_dim}")
+            if l.ff_kind not in ("", "dense", "moe"):
+                raise ValueError(f"layer {i}: unknown feed-forward kind {l.ff_kind!r}")
+            if l.ff_kind == "dense" and l.ff < 1:
+                raise ValueError(f"layer {i}: a dense feed-forward needs its width")
+            if l.ff_kind == "moe" and (not 1 <= l.top <= l.experts or l.expert_ff < 1):
+                raise ValueError(f"layer {i}: top {l.top} of {l.experts} experts of width {l.expert_ff}")
+        if self.loop_times < 0 or (self.loop_times and not 0 <= self.loop_start < self.loop_stop <= len(self.layers)):
+            raise ValueError(f"layers {self.loop_start} .. {self.loop_stop} of {len(self.layers)} cannot run {self.loop_times} times")
+        if self.logit_softcap < 0:
+            raise ValueError("the cap on the logits must be positive (or 0: none)")
+
+    @classmethod
+    def from_dir(cls, path: str) -> "PikadraShape":
+        with open(os.path.join(path, "config.json")) as f:
+            return cls.from_config(json.load(f), name=os.path.basename(os.path.normpath(path)))
+
+    def to_config(self) -> dict:
+        """The ``config.json`` form (what ``from_config`` reads)."""
+        out = []
+        for l in self.layers:
+            mixer = {"dim": l.dim, "heads": l.heads, "kv_rank": l.kv_rank, "q_rank": l.q_rank, "rot_dim": l.rot_dim, "scale": l.scale,
+                     "vdim": l.vdim}
+            if l.rot_dims:
+                mixer["rot"] = {"base": l.rot_base, "dims": l.rot_dims}
+            if l.ff_kind == "dense":
+                mlp = {"ff": l.ff, "kind": "dense"}
+            elif l.ff_kind == "moe":
+                mlp = {"expert": {"ff": l.expert_ff}, "kind": "moe", "router": {"experts": l.experts, "top": l.top}}
+                if l.shared_ff:
+                    mlp["shared"] = {"ff": l.shared_ff}
+            else:
+                mlp = None
+            out.append({"type": l.kind, "mixer": mixer, "mlp": mlp})
+        c = {"architecture": self.ARCHITECTURE, "embedding": {"scale": self.embed_scale}, "layers": out, "logit_scale": self.logit_scale,
+             "norm": {"eps": self.norm_eps}, "vocab": self.vocab_size, "width": self.hidden_size}
+        if self.logit_softcap:
+            c["logit_softcap"] = self.logit_softcap
+        if self.loop_times:
+            c["loop"] = {"start": self.loop_start, "stop": self.loop_stop, "times": self.loop_times}
+        return c
+
+    @classmethod
+    def uniform(cls, vocab: int, width: int, n_layers: int, heads: int, dim: int, rot_dim: int, kv_rank: int, q_rank: int, dense_ff: int = 0,
+                experts: int = 0, top: int = 0, expert_ff: int = 0, shared_ff: int = 0, loop=None, name: str = "pikadra") -> "PikadraShape":
+        """A stack of equal layers: ``experts`` > 0 gives every layer a mixture of experts (with a shared expert if ``shared_ff``), else
+        ``dense_ff`` > 0 a dense feed-forward.  ``loop``: (start, stop, times)."""
+        layers = []
+        for _ in range(n_layers):
+            lay = PikadraLayer(heads=heads, dim=dim, rot_dim=rot_dim, vdim=dim, kv_rank=kv_rank, q_rank=q_rank, scale=(dim + rot_dim) ** -0.5,
+                               rot_base=10000.0, rot_dims=rot_dim)
+            if experts:
+                lay.ff_kind, lay.experts, lay.top, lay.expert_ff, lay.shared_ff = "moe", experts, top, expert_ff, shared_ff
+            elif dense_ff:
+                lay.ff_kind, lay.ff = "dense", dense_ff
+            layers.append(lay)
+        start, stop, times = loop or (0, 0, 0)
+        s = cls(vocab_size=vocab, hidden_size=width, norm_eps=1e-6, layers=layers, embed_scale=width ** 0.5, loop_start=start, loop_stop=stop,
+                loop_times=times, logit_scale=width ** -0.5, logit_softcap=20.0, name=name)
+        s.check()
+        return s
+
+
 def architecture_of(path: str) -> str:
     """Which model family a checkpoint directory holds: ``architecture`` (Kazolorn) or HF's ``model_type``."""
     with open(os.path.join(path, "config.json")) as f:
@@ -867,4 +1032,6 @@ def architecture_of(path: str) -> str:
         return "fivesun"
     if c.get("architecture") == BepepelShape.ARCHITECTURE:
         return "bepepel"
+    if c.get("architecture") == PikadraShape.ARCHITECTURE:
+        return "pikadra"
     return str(c.get("model_type", "llama"))

@@ -620,3 +620,82 @@ def load_bepepel_safetensors(path: str, cfg):
         if tuple(raw[k].shape) != tuple(shp):
             raise ValueError(f"{path}: {k} has shape {tuple(raw[k].shape)}, the configuration implies {tuple(shp)}")
     return {k: raw[k] for k in want}
+
+
+def pikadra_weight_shapes(cfg) -> Dict[str, tuple]:
+    """Tensor names and shapes of a Pikadra checkpoint (``model.safetensors``): ``embed`` (also the output projection); with a loop
+    ``loop.in`` and ``loop.step``; per layer ``l{i}.norm1``, ``l{i}.mix.dq dq.norm uq dkv dkv.norm uk uv sink g o`` and, with a
+    feed-forward, ``l{i}.mlp.gate|up|down`` (dense) or ``l{i}.mlp.router``, ``l{i}.mlp.e{j}.gate|up|down`` and
+    ``l{i}.mlp.shared.gate|up|down|sg``; then ``final.norm``."""
+    W = cfg.hidden_size
+    s = {"embed": (cfg.vocab_size, W)}
+    if cfg.loop_times:
+        s["loop.in"], s["loop.step"] = (W, 2 * W), (cfg.loop_times, W)
+
+    def unit(pre, ff):
+        s[pre + "gate"], s[pre + "up"], s[pre + "down"] = (ff, W), (ff, W), (W, ff)
+
+    for i, l in enumerate(cfg.layers):
+        p, m = f"l{i}.", f"l{i}.mix."
+        s[p + "norm1"] = (W,)
+        s[m + "dq"], s[m + "dq.norm"], s[m + "uq"] = (l.q_rank, W), (l.q_rank,), (l.heads * (l.dim + l.rot_dim), l.q_rank)
+        s[m + "dkv"], s[m + "dkv.norm"] = (l.kv_rank + l.rot_dim, W), (l.kv_rank,)
+        s[m + "uk"], s[m + "uv"] = (l.heads * l.dim, l.kv_rank), (l.heads * l.vdim, l.kv_rank)
+        s[m + "sink"], s[m + "g"], s[m + "o"] = (l.heads,), (l.heads, W), (W, l.heads * l.vdim)
+        if l.ff_kind == "dense":
+            unit(p + "mlp.", l.ff)
+        elif l.ff_kind == "moe":
+            s[p + "mlp.router"] = (l.experts, W)
+            for j in range(l.experts):
+                unit(p + f"mlp.e{j}.", l.expert_ff)
+            if l.shared_ff:
+                unit(p + "mlp.shared.", l.shared_ff)
+                s[p + "mlp.shared.sg"] = (1, W)
+    s["final.norm"] = (W,)
+    return s
+
+
+def make_pikadra_weights(cfg, seed: int = 0, device="cpu", scale: float = 1.0):
+    """Seeded random weights (bfloat16 torch tensors) with nothing at a value that would hide a dropped term: norm weights scattered
+    around zero (model norms) and around one (latent norms), sinks of both signs, step vectors of the stream's own size."""
+    import torch
+    g = torch.Generator(device="cpu").manual_seed(seed)
+    on_gpu = str(device) != "cpu"
+    gd = torch.Generator(device=device).manual_seed(seed) if on_gpu else g
+
+    def rnd(shape, big=False):
+        if big and on_gpu:
+            return torch.randn(shape, generator=gd, device=device, dtype=torch.float32)
+        return torch.randn(shape, generator=g, dtype=torch.float32).to(device)
+
+    out = {}
+    for name, shp in pikadra_weight_shapes(cfg).items():
+        leaf = name.rsplit(".", 1)[-1]
+        if leaf == "norm1" or name == "final.norm":
+            w = 0.2 * rnd(shp)
+        elif leaf == "norm":
+            w = 1.0 + 0.2 * rnd(shp)
+        elif leaf == "sink":
+            w = 1.5 * rnd(shp)
+        elif name == "loop.step":
+            w = 0.5 * rnd(shp)
+        elif leaf == "embed":
+            w = rnd(shp, big=True) / (shp[-1] ** 0.5)
+        else:
+            w = (scale / (shp[-1] ** 0.5)) * rnd(shp, big=True)
+        out[name] = w.to(torch.bfloat16)
+    return out
+
+
+def load_pikadra_safetensors(path: str, cfg):
+    """The tensors of ``<path>/model.safetensors`` by their own names, on the host, checked against the shapes the
+    configuration implies."""
+    raw = read_checkpoint_dir(path)
+    want = pikadra_weight_shapes(cfg)
+    missing = [k for k in want if k not in raw]
+    if missing:
+        raise KeyError(f"{path}: tensors missing for this configuration: {missing[:6]}{' ...' if len(missing) > 6 else ''}")
+    for k, shp in want.items():
+        if tuple(raw[k].shape) != tuple(shp):
+            raise ValueError(f"{path}: {k} has shape {tuple(raw[k].shape)}, the configuration implies {tuple(shp)}")
+    return {k: raw[k] for k in want}
