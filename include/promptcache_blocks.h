@@ -16,7 +16,7 @@
 extern "C" {
 #endif
 
-#define PCB_ABI_VERSION 4
+#define PCB_ABI_VERSION 5
 #define PCB_OK 0
 #define PCB_ERR_ARG (-2001)
 #define PCB_ERR_HIP_BASE (-3000)
@@ -63,13 +63,19 @@ int pcb_mix_norm(const pcb_mix_norm_args* a, void* stream);
  * rows      A row r = row_scale[r] * X[row_src ? row_src[r] : r]   (the scaled row is rounded to E)
  * groups    n_groups > 0: rows [group_off[g], group_off[g+1]) use W + g * w_group_stride (and W2 likewise); M is then an upper
  *           bound of group_off[n_groups] (the launch covers it; the kernel reads the offsets)
+ * batches   n_batch > 0 (instead of groups): n_batch products of M rows each in one launch; product b reads x + b * x_batch_stride and
+ *           W + b * w_group_stride and writes y + b * y_batch_stride (elements; row_src / row_dst apply to each): per-head projections
+ *           of head-by-head row matrices
  * epilogue  PCB_EPI_STORE      v = acc + bias[n]
  *           PCB_EPI_SILU_MUL   v = f(acc + bias[n]) * (acc2 + bias2[n]), acc2 = A W2^T   (gated unit; f = SiLU, or `act` when it is
  *                              PCB_ACT_RELU / PCB_ACT_GELU_TANH / PCB_ACT_SILU; both biases optional)
+ *                              row_gate (E, one number per row, stride ld_row_gate): v *= row_gate[m]
  *           PCB_EPI_SCALE_ADD  v = (base ? base[m][n] : y32[m][n]) + col_scale[n] * (acc + bias[n]), stored fp32 (ldy)
  * output    STORE / SILU_MUL: element type E, or fp32 when out_f32; row m goes to y + (row_dst ? row_dst[m] : m) * ldy.
  *           split_n > 0 (STORE only): columns n >= split_n go to y2 instead: row m at y2 + row_off2[m], column c = n - split_n at
- *           (c / head_dim2) * head_stride2 + c % head_dim2  (a projection that appends its second part to a key cache). */
+ *           (c / head_dim2) * head_stride2 + c % head_dim2  (a projection that appends its second part to a key cache).  y2_f32:
+ *           that part is stored as fp32, row m at y2 + m * head_stride2, row_off2 and head_dim2 unused (router logits that ride in a
+ *           wider projection). */
 #define PCB_EPI_STORE 0
 #define PCB_EPI_SILU_MUL 1
 #define PCB_EPI_SCALE_ADD 2
@@ -123,6 +129,11 @@ typedef struct pcb_linear_args {
     int32_t act2;
     float act_param;   /* PCB_ACT_SOFTCAP: the cap; PCB_ACT_LOGSIGMOID, PCB_ACT_SCALE: the factor (it serves act and act2 alike) */
     const void* bias2; /* [N] E, may be null: the second product's bias of the gated epilogue */
+    int32_t n_batch;
+    int64_t x_batch_stride, y_batch_stride;
+    const void* row_gate;
+    int64_t ld_row_gate;
+    int32_t y2_f32;
 } pcb_linear_args;
 int pcb_linear(const pcb_linear_args* a, void* stream);
 
@@ -380,10 +391,14 @@ int pcb_state_chain(const float* local, float* start, float* state, int64_t slot
 /* A residual step with a norm after the sublayer and the norm before the next one, one workgroup per row, in two optional halves:
  *   write (y given):  t = y[src] * (gate ? gate[src] : 1);  x[src] += post_gain ? t / sqrt(mean(t^2) + eps) * post_gain : t
  *                     (with `rows` the sum is used but not written back)
+ *                     pair (fp32 [.. * pair_top][width]): y[src] + sum_k pair_weight[p] * pair[p], p = src * pair_top + k (fixed order),
+ *                     stands for y[src] (a mixture's experts join in the same pass; y may then be null)
  *   read (out given): out[r] = x[src] / sqrt(mean(x[src]^2) + eps) * gain as E;  x_out[r] = x[src] (fp32) if given
+ *                     gain null: out[r] = x[src] as E, without a norm
  *                     layer_norm: out[r] = (x - mean(x)) / sqrt(mean((x - mean(x))^2) + eps) * gain + bias instead
  * y_scale: the sublayer's result enters as y_scale * y (after gate and post norm; 1 = as it is).
- * src = rows ? rows[r] : r.  y fp32 [..][width]; gate E rows of stride ldg; x fp32 [..][width].  width <= 16384. */
+ * src = rows ? rows[r] : r.  y fp32 [..][width]; gate E rows of stride ldg; x fp32 [..][width]; out rows ldo elements apart (0:
+ * width).  width <= 16384. */
 typedef struct pcb_post_norm_args {
     uint32_t struct_bytes;
     int32_t dtype;
@@ -402,6 +417,10 @@ typedef struct pcb_post_norm_args {
     float y_scale;
     int32_t layer_norm;
     const float* bias; /* [width] fp32, layer_norm only (null: none) */
+    const float* pair;
+    const float* pair_weight;
+    int32_t pair_top;
+    int64_t ldo;
 } pcb_post_norm_args;
 int pcb_post_norm(const pcb_post_norm_args* a, void* stream);
 
@@ -412,9 +431,11 @@ int pcb_post_norm(const pcb_post_norm_args* a, void* stream);
  *   keep:   keep[row][h * head_dim + c] = x                                       (fp32: what a later launch blends with)
  *   rotate: columns rot_off + 2i, rot_off + 2i + 1 (i < rot_dims / 2) turn by the angle pos[row] * freqs[i]:
  *           (u, v) <- rot_mag * (u cos - v sin, v cos + u sin); the angle is a float64 product, other columns pass unchanged
+ *           (rot_half: the pair is columns rot_off + i, rot_off + rot_dims / 2 + i instead)
  *   store:  E at dst + (row_off ? row_off[row] : row * ld_dst) + h * head_stride + c * col_stride  (rows of a matrix, a cache kept
  *           row by row, or one kept column by column)
- * freqs: float64 [rot_dims / 2] on the device, shared by the segments that rotate (they have the same rot_dims).  head_dim <= 1024. */
+ * freqs: float64 [rot_dims / 2] on the device, shared by the segments that rotate (they have the same rot_dims).  head_dim <= 16384,
+ * rot_dims <= 1024.  A segment may work in place (dst = src, the same strides). */
 typedef struct pcb_head_prep_seg {
     const void* src;
     int64_t ld_src;
@@ -442,6 +463,7 @@ typedef struct pcb_head_prep_args {
     const double* freqs;
     float rot_mag;
     float eps;
+    int32_t rot_half;
     pcb_head_prep_seg seg[4];
 } pcb_head_prep_args;
 int pcb_head_prep(const pcb_head_prep_args* a, void* stream);
@@ -530,6 +552,66 @@ typedef struct pcb_gla_args {
     float* ld_sum;
 } pcb_gla_args;
 int pcb_gla(const pcb_gla_args* a, void* stream);
+
+/* Causal softmax attention of prompt rows, tiled through LDS, over keys and values that lie as plain rows (a step's own projections,
+ * or what was rebuilt from a cached latent).  tile t = {base row, first query position, query rows (<= tile_rows), first flat row}
+ * (int32 x 4, device): key j of the request sits in row base + j of k and v, and the rows up to the tile's last query position
+ * exist.  Query head h (column h * dim of its flat row) reads key head h / (H / Hkv).  The last tail_dim of the dim key columns may be
+ * shared by all heads: they then come from row (tail_rows ? tail_rows[base + j] : base + j) of k_tail.  Key j is seen by the query
+ * at position i iff j <= i and (window <= 0 or i - j < window).  sink (fp32 [H]) and gate (E, one number per row and head, stride
+ * ldg): as in pcb_attn_softmax.  tile_rows: 64, or 128 (bf16).  dim <= 256, vdim <= 256. */
+typedef struct pcb_attn_prompt_args {
+    uint32_t struct_bytes;
+    int32_t dtype;
+    const void* q;
+    int64_t ldq;
+    const int32_t* tiles;
+    int32_t n_tiles;
+    int32_t tile_rows;
+    const void* k;
+    int64_t k_row_stride, k_head_stride;
+    const void* k_tail;
+    int64_t tail_row_stride;
+    const int32_t* tail_rows;
+    int32_t tail_dim;
+    const void* v;
+    int64_t v_row_stride, v_head_stride;
+    int32_t H, Hkv, dim, vdim;
+    float scale;
+    int32_t window;
+    const float* sink;
+    const void* gate;
+    int64_t ldg;
+    void* out;
+    int64_t ldo;
+} pcb_attn_prompt_args;
+int pcb_attn_prompt(const pcb_attn_prompt_args* a, void* stream);
+
+/* Causal softmax attention of single rows over one key head whose values are the first vdim columns of the dim-column key rows
+ * themselves (decoding over a shared latent).  tile r = {slot, position, 1, flat row} (int32 x 4, device); key j of slot s: cache +
+ * s * slot_stride + j * row_stride.  q: head h at column h * dim; out: head h at column h * vdim.  window, sink, gate (one number per row
+ * and head), n_splits and part as in pcb_attn_softmax.  dim <= 768, vdim <= 512. */
+typedef struct pcb_attn_latent_args {
+    uint32_t struct_bytes;
+    int32_t dtype;
+    const void* q;
+    int64_t ldq;
+    const int32_t* tiles;
+    int32_t n_rows;
+    const void* cache;
+    int64_t slot_stride, row_stride;
+    int32_t H, dim, vdim;
+    float scale;
+    int32_t window;
+    const float* sink;
+    const void* gate;
+    int64_t ldg;
+    void* out;
+    int64_t ldo;
+    int32_t n_splits;
+    float* part;
+} pcb_attn_latent_args;
+int pcb_attn_latent(const pcb_attn_latent_args* a, void* stream);
 
 #ifdef __cplusplus
 }

@@ -13,41 +13,12 @@
 // one token instead: the heads read the same keys and values, so one pass over them serves sixteen heads.
 // Scores, maxima, weights and sums are fp32.  bf16: the weights enter the second product as a hi + lo pair of bf16 values (two
 // MFMAs), so they are not rounded to 8 bits; fp32: the fp32 matrix cores take them as they are.
-#include "pb_common.h"
+#include "pb_attn_common.h"
 
 namespace {
 using namespace pcb;
 
 constexpr int AW = 4;          // waves of a workgroup
-
-template <typename E>
-struct PFrag;
-template <>
-struct PFrag<bf16_t> {
-    Frag<bf16_t> hi, lo;
-};
-template <>
-struct PFrag<float> {
-    Frag<float> hi;
-};
-
-__device__ __forceinline__ void make_p(PFrag<bf16_t>& f, const float (&p)[8]) {
-    // hi = the upper 16 bits of p as they stand, lo = the rest, cut to 16 bits: hi + lo carries 16 bits of p's mantissa (p is a
-    // finite non-negative weight, so no rounding carry or NaN needs care)
-    uint32_t h[8], l[8];
-#pragma unroll
-    for (int e = 0; e < 8; ++e) {
-        const uint32_t u = __float_as_uint(p[e]);
-        h[e] = u >> 16;
-        l[e] = __float_as_uint(p[e] - __uint_as_float(u & 0xffff0000u)) >> 16;
-    }
-    f.hi.v = u32x4{h[0] | (h[1] << 16), h[2] | (h[3] << 16), h[4] | (h[5] << 16), h[6] | (h[7] << 16)};
-    f.lo.v = u32x4{l[0] | (l[1] << 16), l[2] | (l[3] << 16), l[4] | (l[5] << 16), l[6] | (l[7] << 16)};
-}
-__device__ __forceinline__ void make_p(PFrag<float>& f, const float (&p)[8]) {
-#pragma unroll
-    for (int e = 0; e < 8; ++e) f.hi.v[e] = p[e];
-}
 
 // the value operand of one 16-column block: element e of lane (column c, group g) is V[key(g, e)][c]
 __device__ __forceinline__ Frag<bf16_t> load_v(const bf16_t* const (&rows)[8], int c, bool ok) {
@@ -97,12 +68,6 @@ __device__ __forceinline__ Frag<float> load_v_cols(const float* col, int g, bool
     for (int e = 0; e < 8; ++e) f.v[e] = ((e < 4 ? 4 * g + e : 16 + 4 * g + e - 4) < valid) ? v[e] : 0.0f;
     return f;
 }
-
-__device__ __forceinline__ f4 mma_p(const Frag<bf16_t>& v, const PFrag<bf16_t>& p, f4 c) {
-    c = mma(v, p.hi, c);
-    return mma(v, p.lo, c);
-}
-__device__ __forceinline__ f4 mma_p(const Frag<float>& v, const PFrag<float>& p, f4 c) { return mma(v, p.hi, c); }
 
 // KSQ: 32-element k-steps of the key size; VB: 16-column blocks of the value size
 template <typename E, int KSQ, int VB>

@@ -1,11 +1,12 @@
 // pcb_head_prep: what happens to projected rows between the projection and the attention -- a unit-RMS norm per head (with or
-// without a gain), a blend with another layer's values, rotary positions on neighbouring column pairs, and the store into a row
+// without a gain), a blend with another layer's values, rotary positions on neighbouring column pairs or on halves, and the store into a row
 // matrix or a slot's cache (row by row or column by column).  Up to four segments (queries, keys, values, ...) per launch.
 //
 // One workgroup per (row, segment).  The turn of every column pair depends on the row's position only, so the workgroup first
 // fills a cos / sin table in LDS -- the angle is the float64 product position x frequency, reduced by float64 sincos, so a
 // position in the thousands costs no bits of the angle -- and its waves then take the heads in turn: one pass for the sum of
-// squares, one that norms, blends, turns and stores.  A lane owns neighbouring column pairs, so a rotation never crosses lanes.
+// squares, one that norms, blends, turns and stores.  A lane owns the two columns of a pair, so a rotation never crosses lanes
+// (and a segment may work in place).
 #include "pb_common.h"
 
 namespace {
@@ -32,7 +33,7 @@ __global__ __launch_bounds__(256) void head_prep_kernel(pcb_head_prep_args a) {
     }
     const float lam = s.blend ? s.blend[0] : 0.0f;
     for (int h = wave; h < s.heads; h += waves) {
-        const E* __restrict__ x = (const E*)s.src + row * s.ld_src + (int64_t)h * s.src_head_stride;
+        const E* x = (const E*)s.src + row * s.ld_src + (int64_t)h * s.src_head_stride;
         float inv = 1.0f;
         if (s.norm) {
             float ss = 0.0f;
@@ -46,29 +47,49 @@ __global__ __launch_bounds__(256) void head_prep_kernel(pcb_head_prep_args a) {
         const float* __restrict__ other = s.blend ? s.other + row * s.ld_other + (int64_t)h * D : nullptr;
         float* __restrict__ keep = s.keep ? s.keep + row * s.ld_keep + (int64_t)h * D : nullptr;
         E* dst = (E*)s.dst + (s.row_off ? s.row_off[row] : row * s.ld_dst) + (int64_t)h * s.head_stride;
-        for (int c0 = 2 * lane; c0 < D; c0 += 128) {
+        // a lane owns whole pairs: pair i < np turns by the position; of the columns that do not turn, pair i >= np is the next two
+        // (interleaved rotation: the pairs in memory order, np of them from rot_off on)
+        for (int i0 = lane; 2 * i0 < D + 1; i0 += 64) {
+            int c[2];
+            int i = -1;                                      // which angle, or none
+            if (a.rot_half && np > 0) {
+                if (i0 < np) {
+                    c[0] = s.rot_off + i0;
+                    c[1] = c[0] + np;
+                    i = i0;
+                } else {
+#pragma unroll
+                    for (int e = 0; e < 2; ++e) {
+                        const int k = 2 * (i0 - np) + e;
+                        c[e] = k < s.rot_off ? k : k + 2 * np;
+                    }
+                }
+            } else {
+                c[0] = 2 * i0;
+                c[1] = c[0] + 1;
+                const int k = (c[0] - s.rot_off) >> 1;       // (rot_off is even: a pair never straddles the rotated range's edge)
+                if (c[0] >= s.rot_off && k < np) i = k;
+            }
             float v[2];
 #pragma unroll
             for (int e = 0; e < 2; ++e) {
-                const int c = c0 + e;
                 float t = 0.0f;
-                if (c < D) {
-                    t = to_f32(x[c]) * inv;
-                    if (s.gain) t *= s.gain[c];
-                    if (other) t = (1.0f - lam) * t + lam * other[c];
-                    if (keep) keep[c] = t;
+                if (c[e] < D) {
+                    t = to_f32(x[c[e]]) * inv;
+                    if (s.gain) t *= s.gain[c[e]];
+                    if (other) t = (1.0f - lam) * t + lam * other[c[e]];
+                    if (keep) keep[c[e]] = t;
                 }
                 v[e] = t;
             }
-            const int i = (c0 - s.rot_off) >> 1;
-            if (c0 >= s.rot_off && i < np) {             // (rot_off is even: a pair never straddles the rotated range's edge)
+            if (i >= 0) {
                 const float u = v[0], w = v[1];
                 v[0] = u * cs[i] - w * sn[i];
                 v[1] = w * cs[i] + u * sn[i];
             }
 #pragma unroll
             for (int e = 0; e < 2; ++e)
-                if (c0 + e < D) dst[(int64_t)(c0 + e) * s.col_stride] = from_f32<E>(v[e]);
+                if (c[e] < D) dst[(int64_t)c[e] * s.col_stride] = from_f32<E>(v[e]);
         }
     }
 }
@@ -82,8 +103,8 @@ PCB_EXPORT int pcb_head_prep(const pcb_head_prep_args* a, void* stream) {
     int rot = 0;
     for (int i = 0; i < a->n_segs; ++i) {
         const pcb_head_prep_seg& s = a->seg[i];
-        PCB_REQUIRE(s.heads > 0 && s.head_dim > 0 && s.head_dim <= 1024 && s.src_head_stride >= 0 && s.ld_src >= (int64_t)(s.heads - 1) * s.src_head_stride + s.head_dim && s.col_stride > 0,
-                    PCB_ERR_ARG, "pcb_head_prep: bad segment sizes (heads of up to 1024 columns)");
+        PCB_REQUIRE(s.heads > 0 && s.head_dim > 0 && s.head_dim <= 16384 && s.src_head_stride >= 0 && s.ld_src >= (int64_t)(s.heads - 1) * s.src_head_stride + s.head_dim && s.col_stride > 0,
+                    PCB_ERR_ARG, "pcb_head_prep: bad segment sizes (heads of up to 16384 columns)");
         PCB_REQUIRE(s.rot_dims >= 0 && s.rot_dims % 2 == 0 && s.rot_off >= 0 && s.rot_off % 2 == 0 && s.rot_off + s.rot_dims <= s.head_dim &&
                         s.rot_dims <= 2 * MAX_PAIRS && (s.rot_dims == 0 || rot == 0 || rot == s.rot_dims),
                     PCB_ERR_ARG, "pcb_head_prep: rotated columns come in pairs inside the head, the same number in every segment that rotates");

@@ -66,7 +66,10 @@ __device__ __forceinline__ void emit(const pcb_linear_args& a, int m, int n, flo
     if (EPI == PCB_EPI_STORE && (a.act | a.act2) && !(a.split_n > 0 && n >= a.split_n) && !(a.split_n3 > 0 && n >= a.split_n3))
         // (the split-off parts are stored as they are)
         v = apply_act((a.act_split > 0 && n >= a.act_split) ? a.act2 : a.act, v, a.act_param);
-    if (EPI == PCB_EPI_SILU_MUL) v = apply_act(a.act == PCB_ACT_NONE ? PCB_ACT_SILU : a.act, v, 0.0f) * (acc2 + bv2);
+    if (EPI == PCB_EPI_SILU_MUL) {
+        v = apply_act(a.act == PCB_ACT_NONE ? PCB_ACT_SILU : a.act, v, 0.0f) * (acc2 + bv2);
+        if (a.row_gate) v *= to_f32(((const E*)a.row_gate)[m * a.ld_row_gate]);
+    }
     if (EPI == PCB_EPI_SCALE_ADD) {
         float* y = (float*)a.y + (int64_t)m * a.ldy + n;
         const float b0 = a.base ? a.base[(int64_t)m * a.ldbase + n] : *y;
@@ -79,11 +82,15 @@ __device__ __forceinline__ void emit(const pcb_linear_args& a, int m, int n, flo
     }
     if (a.split_n > 0 && n >= a.split_n) {
         const int c = n - a.split_n;
+        if (a.y2_f32) {
+            ((float*)a.y2)[m * a.head_stride2 + c] = v;
+            return;
+        }
         E* y = (E*)a.y2 + a.row_off2[m] + (int64_t)(c / a.head_dim2) * a.head_stride2 + c % a.head_dim2;
         *y = from_f32<E>(v);
         return;
     }
-    const int64_t at = (int64_t)(a.row_dst ? a.row_dst[m] : m) * a.ldy + n;
+    const int64_t at = (int64_t)(a.row_dst ? a.row_dst[m] : m) * a.ldy + n + (a.n_batch > 0 ? (int64_t)blockIdx.z * a.y_batch_stride : 0);
     if (a.out_f32)
         ((float*)a.y)[at] = v;
     else
@@ -122,12 +129,13 @@ __global__ __launch_bounds__(256) void linear_kernel(pcb_linear_args a) {
     } else {
         m_lo = blockIdx.y * BM;
         m_hi = a.M;
+        if (a.n_batch > 0) g = blockIdx.z;
         if (m_lo >= m_hi) return;
     }
     const int n_lo = blockIdx.x * BN;
     const E* W = (const E*)a.w + (int64_t)g * a.w_group_stride;
     const E* W2 = TWO ? (const E*)a.w2 + (int64_t)g * a.w_group_stride : nullptr;
-    const E* X = (const E*)a.x;
+    const E* X = (const E*)a.x + (a.n_batch > 0 ? (int64_t)blockIdx.z * a.x_batch_stride : 0);
     const bool vec = (K % CE == 0) && (a.ldx % CE == 0) && (a.ldw % CE == 0) && (((uintptr_t)X | (uintptr_t)W | (uintptr_t)W2) % 16 == 0);
     const bool scaled = a.row_scale != nullptr;
 
@@ -275,12 +283,13 @@ __global__ __launch_bounds__(64 * SKW) void linear_skinny_kernel(pcb_linear_args
     } else {
         m_lo = blockIdx.y * 16;
         m_hi = a.M;
+        if (a.n_batch > 0) g = blockIdx.z;
         if (m_lo >= m_hi) return;
     }
     const int n_lo = blockIdx.x * 16;
     const E* W = (const E*)a.w + (int64_t)g * a.w_group_stride;
     const E* W2 = TWO ? (const E*)a.w2 + (int64_t)g * a.w_group_stride : nullptr;
-    const E* X = (const E*)a.x;
+    const E* X = (const E*)a.x + (a.n_batch > 0 ? (int64_t)blockIdx.z * a.x_batch_stride : 0);
     const bool vec = (K % CE == 0) && (a.ldx % CE == 0) && (a.ldw % CE == 0) && (((uintptr_t)X | (uintptr_t)W | (uintptr_t)W2) % 16 == 0);
     const int n_b = n_lo + l15, m_a = m_lo + l15;
     const bool b_ok = n_b < N, a_ok = m_a < m_hi;
@@ -330,7 +339,7 @@ __global__ __launch_bounds__(64 * SKW) void linear_skinny_kernel(pcb_linear_args
 template <typename E, int EPI, int TM, int TN>
 int launch(const pcb_linear_args& a, hipStream_t stream) {
     constexpr int BM = 32 * TM, BN = 32 * TN;
-    const dim3 grid(pcb_ceil_div(a.N, BN), pcb_ceil_div(a.M, BM) + (a.n_groups > 0 ? a.n_groups : 0));
+    const dim3 grid(pcb_ceil_div(a.N, BN), pcb_ceil_div(a.M, BM) + (a.n_groups > 0 ? a.n_groups : 0), a.n_batch > 0 ? a.n_batch : 1);
     hipLaunchKernelGGL((linear_kernel<E, EPI, TM, TN>), grid, dim3(256), 0, stream, a);
     return pcb_check_launch("linear_kernel");
 }
@@ -343,7 +352,7 @@ int dispatch(const pcb_linear_args& a, hipStream_t stream) {
     // workgroups on the chip, each walking all of K)
     const bool big = rows > 64 && a.N > 64;
     if (rows <= 16) {
-        const dim3 grid(pcb_ceil_div(a.N, 16), pcb_ceil_div(a.M, 16) + (a.n_groups > 0 ? a.n_groups : 0));
+        const dim3 grid(pcb_ceil_div(a.N, 16), pcb_ceil_div(a.M, 16) + (a.n_groups > 0 ? a.n_groups : 0), a.n_batch > 0 ? a.n_batch : 1);
         switch (a.epilogue) {
             case PCB_EPI_STORE:
                 hipLaunchKernelGGL((linear_skinny_kernel<E, PCB_EPI_STORE>), grid, dim3(64 * SKW), 0, stream, a);
@@ -384,12 +393,20 @@ PCB_EXPORT int pcb_linear(const pcb_linear_args* a, void* stream) {
     if (a->M == 0) return PCB_OK;
     PCB_REQUIRE(a->x && a->w && a->y, PCB_ERR_ARG, "pcb_linear: null pointer");
     PCB_REQUIRE(a->n_groups >= 0 && (a->n_groups == 0 || a->group_off), PCB_ERR_ARG, "pcb_linear: groups need their offsets");
+    PCB_REQUIRE(a->n_batch >= 0 && a->n_batch <= 65535 &&
+                    (a->n_batch == 0 || (a->n_groups == 0 && a->epilogue == PCB_EPI_STORE && a->split_n == 0 && a->split_n3 == 0 && !a->bias &&
+                                         !a->row_scale && a->x_batch_stride >= 0 && a->y_batch_stride >= 0 && a->w_group_stride >= 0)),
+                PCB_ERR_ARG, "pcb_linear: a batch goes with plain stores (no groups, no split destinations, no bias)");
+    PCB_REQUIRE(!a->row_gate || (a->epilogue == PCB_EPI_SILU_MUL && a->n_groups == 0 && a->ld_row_gate >= 1), PCB_ERR_ARG,
+                "pcb_linear: a gate per row goes with the gated epilogue of a plain (ungrouped) launch");
     PCB_REQUIRE(a->epilogue != PCB_EPI_SILU_MUL || a->w2, PCB_ERR_ARG, "pcb_linear: the gated epilogue takes w2");
     PCB_REQUIRE(a->epilogue == PCB_EPI_SILU_MUL || !a->bias2, PCB_ERR_ARG, "pcb_linear: a second bias goes with the gated epilogue");
     PCB_REQUIRE(a->epilogue != PCB_EPI_SCALE_ADD || (a->col_scale && a->ldy >= a->N && !a->row_dst), PCB_ERR_ARG,
                 "pcb_linear: scale-add needs col_scale and a plain fp32 destination");
     PCB_REQUIRE(a->split_n == 0 || (a->epilogue == PCB_EPI_STORE && a->split_n > 0 && a->split_n < a->N && a->y2 && a->row_off2 &&
-                                    a->head_dim2 > 0 && a->ldy >= a->split_n),
+                                    a->head_dim2 > 0 && a->ldy >= a->split_n) ||
+                    (a->epilogue == PCB_EPI_STORE && a->split_n > 0 && a->split_n < a->N && a->y2 && a->y2_f32 && a->split_n3 == 0 &&
+                     a->n_groups == 0 && a->head_stride2 >= a->N - a->split_n && a->ldy >= a->split_n),
                 PCB_ERR_ARG, "pcb_linear: bad split destination");
     PCB_REQUIRE(a->split_n3 == 0 || (a->epilogue == PCB_EPI_STORE && a->split_n3 > a->split_n && a->split_n3 < a->N && a->y3 && a->row_off3 &&
                                      a->col_stride3 > 0 && (a->split_n > 0 || a->ldy >= a->split_n3)),

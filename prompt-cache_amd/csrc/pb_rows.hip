@@ -438,11 +438,16 @@ __global__ __launch_bounds__(1024) void post_norm_kernel(pcb_post_norm_args a) {
     const int64_t src = a.rows ? a.rows[r] : r;
     float* __restrict__ x = a.x + src * W;
     float ss[1] = {0.0f};
-    if (a.y) {
-        const float* __restrict__ y = a.y + src * W;
+    if (a.y || a.pair) {
+        const float* __restrict__ y = a.y ? a.y + src * W : nullptr;
         const E* __restrict__ g = a.gate ? (const E*)a.gate + src * a.ldg : nullptr;
+        const float* __restrict__ pair = a.pair ? a.pair + src * a.pair_top * W : nullptr;
+        const float* __restrict__ pw = a.pair ? a.pair_weight + src * a.pair_top : nullptr;
         for (int c = threadIdx.x; c < W; c += blockDim.x) {
-            const float t = y[c] * (g ? to_f32(g[c]) : 1.0f);
+            float t = y ? y[c] : 0.0f;
+            if (pair)
+                for (int k = 0; k < a.pair_top; ++k) t += pw[k] * pair[(int64_t)k * W + c];
+            t *= g ? to_f32(g[c]) : 1.0f;
             row[c] = t;
             ss[0] += t * t;
         }
@@ -469,7 +474,11 @@ __global__ __launch_bounds__(1024) void post_norm_kernel(pcb_post_norm_args a) {
     if (a.x_out)
         for (int c = threadIdx.x; c < W; c += blockDim.x) a.x_out[(int64_t)r * W + c] = row[c];
     if (!a.out) return;
-    E* o = (E*)a.out + (int64_t)r * W;
+    E* o = (E*)a.out + (int64_t)r * (a.ldo > 0 ? a.ldo : W);
+    if (!a.gain) {
+        for (int c = threadIdx.x; c < W; c += blockDim.x) o[c] = from_f32<E>(row[c]);
+        return;
+    }
     if (a.layer_norm) {
         // mean first, then the mean of the squared deviations (the row waits in LDS; a thread meets its own columns again)
         float sm[1] = {0.0f};
@@ -704,8 +713,10 @@ PCB_EXPORT int pcb_post_norm(const pcb_post_norm_args* a, void* stream) {
     PCB_REQUIRE(PCB_DTYPE_OK(a->dtype) && a->n_rows >= 0 && a->width > 0 && a->width <= 16384, PCB_ERR_ARG,
                 "pcb_post_norm: bad sizes (width <= 16384)");
     if (a->n_rows == 0) return PCB_OK;
-    PCB_REQUIRE(a->x && (!a->out || a->gain) && (!a->gate || (a->y && a->ldg >= a->width)) && (!a->post_gain || a->y), PCB_ERR_ARG,
-                "pcb_post_norm: null pointer (a gate and a norm after the sublayer need its result, a norm its gain)");
+    PCB_REQUIRE(a->x && (!a->layer_norm || !a->out || a->gain) && (!a->gate || (a->y && a->ldg >= a->width)) && (!a->post_gain || a->y),
+                PCB_ERR_ARG, "pcb_post_norm: null pointer (a gate and a norm after the sublayer need its result, a norm its gain)");
+    PCB_REQUIRE((!a->pair || (a->pair_weight && a->pair_top > 0)) && (a->ldo == 0 || a->ldo >= a->width), PCB_ERR_ARG,
+                "pcb_post_norm: pairs need their weights and their number per row; output rows may not overlap");
     const size_t lds = (size_t)a->width * sizeof(float);
     const dim3 threads(a->n_rows <= 512 && a->width > 1024 ? 1024 : 256);
     if (a->dtype == PCB_BF16)

@@ -19,7 +19,7 @@ EPI_STORE, EPI_SILU_MUL, EPI_SCALE_ADD = 0, 1, 2
 ACT_NONE, ACT_SILU, ACT_SIGMOID, ACT_RELU2, ACT_SOFTPLUS, ACT_SOFTCAP, ACT_RELU, ACT_GELU_TANH, ACT_LOGSIGMOID, ACT_SCALE = range(10)
 NORM_NONE, NORM_RMS, NORM_DYT = 0, 1, 2
 SCORE_SIGMOID, SCORE_SOFTMAX = 0, 1
-ABI_VERSION = 4
+ABI_VERSION = 5
 DTYPES = {torch.bfloat16: BF16, torch.float32: F32}
 
 
@@ -42,7 +42,9 @@ class LinearArgs(C.Structure):
                 ("base", _vp), ("ldbase", _i64), ("col_scale", _vp),
                 ("split_n", _i32), ("y2", _vp), ("row_off2", _vp), ("head_dim2", _i32), ("head_stride2", _i64),
                 ("split_n3", _i32), ("y3", _vp), ("row_off3", _vp), ("col_stride3", _i64),
-                ("act", _i32), ("act_split", _i32), ("act2", _i32), ("act_param", _f32), ("bias2", _vp)]
+                ("act", _i32), ("act_split", _i32), ("act2", _i32), ("act_param", _f32), ("bias2", _vp),
+                ("n_batch", _i32), ("x_batch_stride", _i64), ("y_batch_stride", _i64), ("row_gate", _vp), ("ld_row_gate", _i64),
+                ("y2_f32", _i32)]
 
 
 class AttnTalkArgs(C.Structure):
@@ -97,7 +99,8 @@ class PostNormArgs(C.Structure):
     _fields_ = [("struct_bytes", C.c_uint32), ("dtype", _i32),
                 ("x", _vp), ("y", _vp), ("gate", _vp), ("ldg", _i64), ("post_gain", _vp), ("gain", _vp),
                 ("out", _vp), ("x_out", _vp), ("rows", _vp), ("eps", _f32), ("n_rows", _i32), ("width", _i32),
-                ("y_scale", _f32), ("layer_norm", _i32), ("bias", _vp)]
+                ("y_scale", _f32), ("layer_norm", _i32), ("bias", _vp),
+                ("pair", _vp), ("pair_weight", _vp), ("pair_top", _i32), ("ldo", _i64)]
 
 
 class HeadPrepSeg(C.Structure):
@@ -111,7 +114,7 @@ class HeadPrepSeg(C.Structure):
 class HeadPrepArgs(C.Structure):
     """``pcb_head_prep_args`` (field for field)."""
     _fields_ = [("struct_bytes", C.c_uint32), ("dtype", _i32), ("n_rows", _i32), ("n_segs", _i32),
-                ("pos", _vp), ("freqs", _vp), ("rot_mag", _f32), ("eps", _f32), ("seg", HeadPrepSeg * 4)]
+                ("pos", _vp), ("freqs", _vp), ("rot_mag", _f32), ("eps", _f32), ("rot_half", _i32), ("seg", HeadPrepSeg * 4)]
 
 
 class MlstmArgs(C.Structure):
@@ -131,6 +134,26 @@ class GlaArgs(C.Structure):
                 ("ld", _vp), ("ldld", _i64), ("dcols", _i32), ("ld_coef", _vp), ("v_scale", _vp), ("ldvs", _i64),
                 ("reqs", _vp), ("n_reqs", _i32), ("state", _vp), ("slot_stride", _i64),
                 ("H", _i32), ("Hk", _i32), ("dim", _i32), ("vdim", _i32), ("q_scale", _f32), ("out", _vp), ("ldo", _i64), ("ld_sum", _vp)]
+
+
+class AttnPromptArgs(C.Structure):
+    """``pcb_attn_prompt_args`` (field for field)."""
+    _fields_ = [("struct_bytes", C.c_uint32), ("dtype", _i32),
+                ("q", _vp), ("ldq", _i64), ("tiles", _vp), ("n_tiles", _i32), ("tile_rows", _i32),
+                ("k", _vp), ("k_row_stride", _i64), ("k_head_stride", _i64),
+                ("k_tail", _vp), ("tail_row_stride", _i64), ("tail_rows", _vp), ("tail_dim", _i32),
+                ("v", _vp), ("v_row_stride", _i64), ("v_head_stride", _i64),
+                ("H", _i32), ("Hkv", _i32), ("dim", _i32), ("vdim", _i32), ("scale", _f32), ("window", _i32),
+                ("sink", _vp), ("gate", _vp), ("ldg", _i64), ("out", _vp), ("ldo", _i64)]
+
+
+class AttnLatentArgs(C.Structure):
+    """``pcb_attn_latent_args`` (field for field)."""
+    _fields_ = [("struct_bytes", C.c_uint32), ("dtype", _i32),
+                ("q", _vp), ("ldq", _i64), ("tiles", _vp), ("n_rows", _i32),
+                ("cache", _vp), ("slot_stride", _i64), ("row_stride", _i64),
+                ("H", _i32), ("dim", _i32), ("vdim", _i32), ("scale", _f32), ("window", _i32),
+                ("sink", _vp), ("gate", _vp), ("ldg", _i64), ("out", _vp), ("ldo", _i64), ("n_splits", _i32), ("part", _vp)]
 
 
 # name -> (restype, argtypes); mirrors include/promptcache_blocks.h one to one
@@ -163,6 +186,8 @@ SIGNATURES = {
     "pcb_mlstm": (C.c_int, [C.POINTER(MlstmArgs), _vp]),
     "pcb_mlstm_chain": (C.c_int, [_vp, _vp, _vp, _vp, _i64, _vp, _i32, _i32, _i32, _i32, _vp]),
     "pcb_gla": (C.c_int, [C.POINTER(GlaArgs), _vp]),
+    "pcb_attn_prompt": (C.c_int, [C.POINTER(AttnPromptArgs), _vp]),
+    "pcb_attn_latent": (C.c_int, [C.POINTER(AttnLatentArgs), _vp]),
 }
 
 
@@ -216,6 +241,11 @@ def _want(t: Optional[torch.Tensor], dtype, what: str) -> None:
         raise TypeError(f"{what}: need a contiguous {dtype} device tensor, got {t.dtype} on {t.device} (contiguous={t.is_contiguous()})")
 
 
+def _reach(t: torch.Tensor) -> int:
+    """Elements from the tensor's first one to the end of its storage: what a strided view may address."""
+    return t.untyped_storage().nbytes() // t.element_size() - t.storage_offset()
+
+
 # ---- wrappers: shapes are checked here, on the host, before the library sees a pointer ---------------------------------------
 def embed_rows(table: torch.Tensor, ids: torch.Tensor, out: torch.Tensor) -> None:
     n, width = out.shape
@@ -263,10 +293,13 @@ def linear(x: torch.Tensor, w: torch.Tensor, y: torch.Tensor, *, M: int, epilogu
            split_n: int = 0, y2=None, row_off2=None, head_dim2: int = 0, head_stride2: int = 0, split_n3: int = 0, y3=None,
            row_off3=None, col_stride3: int = 0, act: int = ACT_NONE,
            act_split: int = 0, act2: int = ACT_NONE, act_param: float = 0.0, ldy: Optional[int] = None, bias2=None,
-           ldx: Optional[int] = None) -> None:
+           ldx: Optional[int] = None, n_batch: int = 0, x_batch_stride: int = 0, y_batch_stride: int = 0, row_gate=None,
+           ld_row_gate: int = 1, y2_f32: bool = False) -> None:
     """``w``: [N, K], or [groups, N, K] with ``group_off``.  ``x``: [rows, K] of the weights' element type.  ``act`` (and ``act2``
     from column ``act_split`` on): the element-wise function of a plain store.  ``ldy``: row stride of ``y`` when it is a
-    column block of a wider matrix."""
+    column block of a wider matrix.  ``n_batch``: that many products at once, ``w`` [n_batch, N, K], their inputs / outputs
+    ``x_batch_stride`` / ``y_batch_stride`` elements apart (``ldx`` / ``ldy`` given).  ``row_gate``: E, one factor per row of the gated
+    epilogue.  ``y2_f32``: the columns from ``split_n`` on go to the fp32 rows ``y2`` (stride ``head_stride2``)."""
     code = _code(w)
     assert x.dtype == w.dtype and (x.is_contiguous() or ldx is not None) and w.is_contiguous() and x.is_cuda and w.is_cuda
     N, K = w.shape[-2], w.shape[-1]
@@ -274,6 +307,11 @@ def linear(x: torch.Tensor, w: torch.Tensor, y: torch.Tensor, *, M: int, epilogu
     if n_groups:
         assert w.dim() == 3 and w.shape[0] == n_groups and group_off is not None and group_off.numel() == n_groups + 1
         _want(group_off, torch.int32, "linear group_off")
+    elif n_batch:
+        assert w.dim() == 3 and w.shape[0] == n_batch and ldx is not None and ldy is not None
+        # (with row tables the rows' own range is the caller's, as everywhere)
+        assert _reach(x) >= (n_batch - 1) * x_batch_stride + (0 if row_src is not None else (M - 1) * ldx) + K
+        assert _reach(y) >= (n_batch - 1) * y_batch_stride + (0 if row_dst is not None else (M - 1) * ldy) + N
     else:
         assert w.dim() == 2
     if w2 is not None:
@@ -288,8 +326,10 @@ def linear(x: torch.Tensor, w: torch.Tensor, y: torch.Tensor, *, M: int, epilogu
     if row_scale is not None:
         _want(row_scale, torch.float32, "linear row_scale")
         assert row_scale.numel() >= M
-    if row_src is None:
+    if row_src is None and not n_batch:
         assert x.shape[0] >= M
+    if row_gate is not None:
+        assert row_gate.dtype == w.dtype and row_gate.is_cuda and _reach(row_gate) >= (M - 1) * ld_row_gate + 1
     out_f32 = int(y.dtype == torch.float32 and (code == BF16 or epilogue == EPI_SCALE_ADD))
     if epilogue == EPI_SCALE_ADD:
         _want(y, torch.float32, "linear y"); _want(col_scale, torch.float32, "linear col_scale")
@@ -297,20 +337,27 @@ def linear(x: torch.Tensor, w: torch.Tensor, y: torch.Tensor, *, M: int, epilogu
         if base is not None:
             _want(base, torch.float32, "linear base")
             assert base.shape[-1] == N and base.shape[0] >= M
+    elif n_batch:
+        assert y.dtype == w.dtype or y.dtype == torch.float32
     else:
-        assert y.is_contiguous() and (y.dtype == w.dtype or y.dtype == torch.float32)
+        assert (y.is_contiguous() or (ldy is not None and row_dst is None and _reach(y) >= (M - 1) * ldy + min(N, split_n or N))) and \
+            (y.dtype == w.dtype or y.dtype == torch.float32)
         cols = split_n if split_n else (split_n3 if split_n3 else N)
         assert (y.shape[-1] == cols or (ldy is not None and ldy >= cols)) and (row_dst is not None or y.shape[0] >= M)
-    if split_n:
+    if y2_f32:
+        _want(y2, torch.float32, "linear y2")
+        assert 0 < split_n < N and head_stride2 >= N - split_n and y2.numel() >= (M - 1) * head_stride2 + N - split_n
+    elif split_n:
         _want(row_off2, torch.int64, "linear row_off2")
         assert y2 is not None and y2.dtype == w.dtype and row_off2.numel() >= M and head_dim2 > 0
     if split_n3:
         _want(row_off3, torch.int64, "linear row_off3")
         assert y3 is not None and y3.dtype == w.dtype and row_off3.numel() >= M and col_stride3 > 0 and split_n3 > split_n
     a = LinearArgs(C.sizeof(LinearArgs), code, epilogue, _p(x), K if ldx is None else ldx, _p(row_src), _p(row_scale), _p(w), _p(w2), K, _p(bias),
-                   M, N, K, _p(group_off), n_groups, N * K if n_groups else 0, _p(y), y.shape[-1] if ldy is None else ldy, out_f32,
+                   M, N, K, _p(group_off), n_groups, N * K if (n_groups or n_batch) else 0, _p(y), y.shape[-1] if ldy is None else ldy, out_f32,
                    _p(row_dst), _p(base), N, _p(col_scale), split_n, _p(y2), _p(row_off2), head_dim2, head_stride2,
-                   split_n3, _p(y3), _p(row_off3), col_stride3, int(act), int(act_split), int(act2), float(act_param), _p(bias2))
+                   split_n3, _p(y3), _p(row_off3), col_stride3, int(act), int(act_split), int(act2), float(act_param), _p(bias2),
+                   n_batch, x_batch_stride, y_batch_stride, _p(row_gate), ld_row_gate, int(y2_f32))
     check(load().pcb_linear(C.byref(a), _stream()), "pcb_linear")
 
 
@@ -560,11 +607,14 @@ def state_chain(local: torch.Tensor, start: torch.Tensor, state: torch.Tensor, c
 
 # ---- sublayers between two norms, per-head preparation, matrix memories ----------------------------------------------------------
 def post_norm(x: torch.Tensor, *, y=None, gate=None, ldg: int = 0, post_gain=None, gain=None, out=None, x_out=None, rows=None,
-              eps: float = 1e-6, n_rows: Optional[int] = None, y_scale: float = 1.0, layer_norm: bool = False, bias=None) -> None:
+              eps: float = 1e-6, n_rows: Optional[int] = None, y_scale: float = 1.0, layer_norm: bool = False, bias=None,
+              pair=None, pair_weight=None, pair_top: int = 0, ldo: int = 0) -> None:
     """``x`` fp32 [T, W] (the residual).  With ``y`` (fp32 [T, W]): x += norm(y * gate) * post_gain (``gate`` E rows of stride
     ``ldg``; without ``post_gain`` the gated y is added as it is).  With ``out`` (E): out = norm(x) * gain, for the rows ``rows``
     only if given (then x itself is not rewritten); ``x_out`` fp32 receives those rows of x.  ``y_scale``: the factor on what is
-    added to x; ``layer_norm``: out = (x - mean) / sqrt(variance + eps) * gain + bias instead of the RMS form."""
+    added to x; ``layer_norm``: out = (x - mean) / sqrt(variance + eps) * gain + bias instead of the RMS form.
+    ``pair`` fp32 [T * pair_top, W] with ``pair_weight``: sum_k weight * pair row joins ``y`` (or stands for it).  Without ``gain``,
+    ``out`` = x as E; ``ldo``: its row stride when it is a column block of a wider matrix."""
     _want(x, torch.float32, "post_norm x"); _want(bias, torch.float32, "post_norm bias")
     assert bias is None or (layer_norm and bias.numel() == x.shape[-1])
     T, W = x.shape
@@ -578,15 +628,20 @@ def post_norm(x: torch.Tensor, *, y=None, gate=None, ldg: int = 0, post_gain=Non
         assert y is not None and gate.is_cuda and ldg >= W and gate.dtype in DTYPES
     code = _code(out) if out is not None else (_code(gate) if gate is not None else BF16)
     if out is not None:
-        assert out.is_contiguous() and out.shape[-1] == W and out.numel() >= n * W and gain is not None and gain.numel() == W
+        assert (out.is_contiguous() and out.shape[-1] == W and out.numel() >= n * W) or (ldo >= W and _reach(out) >= (n - 1) * ldo + W)
+        assert gain is None or gain.numel() == W
         assert gate is None or gate.dtype == out.dtype
     assert post_gain is None or post_gain.numel() == W
+    if pair is not None:
+        _want(pair, torch.float32, "post_norm pair"); _want(pair_weight, torch.float32, "post_norm pair_weight")
+        assert pair_top > 0 and pair.shape[-1] == W and pair.shape[0] >= (T if rows is not None else n) * pair_top
+        assert pair_weight.numel() >= (T if rows is not None else n) * pair_top
     if x_out is not None:
         assert x_out.numel() >= n * W
     if rows is not None:
         _want(rows, torch.int32, "post_norm rows")
     a = PostNormArgs(C.sizeof(PostNormArgs), code, _p(x), _p(y), _p(gate), ldg, _p(post_gain), _p(gain), _p(out), _p(x_out), _p(rows),
-                     float(eps), n, W, float(y_scale), int(layer_norm), _p(bias))
+                     float(eps), n, W, float(y_scale), int(layer_norm), _p(bias), _p(pair), _p(pair_weight), pair_top, ldo)
     check(load().pcb_post_norm(C.byref(a), _stream()), "pcb_post_norm")
 
 
@@ -612,13 +667,14 @@ def head_seg(src: torch.Tensor, ld_src: int, heads: int, head_dim: int, dst: tor
 
 
 def head_prep(segs, n_rows: int, dtype, *, pos: Optional[torch.Tensor] = None, freqs: Optional[torch.Tensor] = None, rot_mag: float = 1.0,
-              eps: float = 1e-6) -> None:
-    """``segs``: one to four ``head_seg`` records; ``pos`` int32 [rows]; ``freqs`` float64 [rot_dims / 2]."""
+              eps: float = 1e-6, rot_half: bool = False) -> None:
+    """``segs``: one to four ``head_seg`` records; ``pos`` int32 [rows]; ``freqs`` float64 [rot_dims / 2];
+    ``rot_half``: column i turns with column i + rot_dims / 2 instead of its neighbour."""
     _want(pos, torch.int32, "head_prep pos"); _want(freqs, torch.float64, "head_prep freqs")
     assert 1 <= len(segs) <= 4
     rot = {s.rot_dims for s in segs if s.rot_dims}
     assert len(rot) <= 1 and (not rot or (pos is not None and freqs is not None and pos.numel() >= n_rows and 2 * freqs.numel() == rot.pop()))
-    a = HeadPrepArgs(C.sizeof(HeadPrepArgs), DTYPES[dtype], n_rows, len(segs), _p(pos), _p(freqs), float(rot_mag), float(eps))
+    a = HeadPrepArgs(C.sizeof(HeadPrepArgs), DTYPES[dtype], n_rows, len(segs), _p(pos), _p(freqs), float(rot_mag), float(eps), int(rot_half))
     for i, sg in enumerate(segs):
         a.seg[i] = sg
     check(load().pcb_head_prep(C.byref(a), _stream()), "pcb_head_prep")
@@ -686,3 +742,36 @@ def gla(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, ld: torch.Tensor, lds
                 int(ldvs), _p(reqs), n_reqs, _p(state), H * dim * vdim, H, Hk, dim, vdim, float(q_scale), _p(out),
                 H * vdim if out is not None else 0, _p(ld_sum))
     check(load().pcb_gla(C.byref(a), _stream()), "pcb_gla")
+
+
+# ---- attention over rows rebuilt from a latent (prompts) and over the latent itself (decoding) -----------------------------------------
+def attn_prompt(q: torch.Tensor, tiles: torch.Tensor, n_tiles: int, tile_rows: int, k: torch.Tensor, k_strides, v: torch.Tensor, v_strides,
+                H: int, Hkv: int, dim: int, vdim: int, scale: float, out: torch.Tensor, *, ldo: int, ldq: Optional[int] = None, k_tail=None,
+                tail_row_stride: int = 0, tail_rows=None, tail_dim: int = 0, window: int = 0, sink=None, gate=None, ldg: int = 0) -> None:
+    """``k_strides`` / ``v_strides``: (row, head) strides in elements of the key and value rows; ``tail_rows``: int32 row of ``k_tail`` per
+    key row; ``gate``: E, one number per row and head."""
+    _want(tiles, torch.int32, "attn_prompt tiles"); _want(sink, torch.float32, "attn_prompt sink"); _want(tail_rows, torch.int32, "attn_prompt tail_rows")
+    assert q.dtype == k.dtype == v.dtype == out.dtype and q.is_cuda and k.is_cuda and v.is_cuda and out.is_cuda
+    ldq = q.shape[-1] if ldq is None else ldq
+    assert tiles.numel() >= 4 * n_tiles and ldq >= H * dim and ldo >= H * vdim and (sink is None or sink.numel() >= H)
+    assert tail_dim == 0 or (k_tail is not None and k_tail.dtype == q.dtype and tail_row_stride >= tail_dim)
+    assert gate is None or (gate.dtype == q.dtype and ldg >= H)
+    a = AttnPromptArgs(C.sizeof(AttnPromptArgs), _code(q), _p(q), ldq, _p(tiles), n_tiles, tile_rows, _p(k), k_strides[0], k_strides[1],
+                       _p(k_tail), tail_row_stride, _p(tail_rows), tail_dim, _p(v), v_strides[0], v_strides[1], H, Hkv, dim, vdim, float(scale),
+                       int(window), _p(sink), _p(gate), ldg, _p(out), ldo)
+    check(load().pcb_attn_prompt(C.byref(a), _stream()), "pcb_attn_prompt")
+
+
+def attn_latent(q: torch.Tensor, tiles: torch.Tensor, n_rows: int, cache: torch.Tensor, slot_stride: int, row_stride: int, H: int, dim: int,
+                vdim: int, scale: float, out: torch.Tensor, *, window: int = 0, sink=None, gate=None, ldg: int = 0, n_splits: int = 1,
+                part=None) -> None:
+    """``q`` E [rows, H * dim]; ``cache``: slots of rows whose first ``vdim`` columns are the value; ``tiles`` int32 {slot, position, 1,
+    flat row} per row; ``part`` fp32 of ``attn_softmax_part(rows, H, n_splits, vdim)`` floats when the keys are cut into runs."""
+    _want(tiles, torch.int32, "attn_latent tiles"); _want(sink, torch.float32, "attn_latent sink"); _want(part, torch.float32, "attn_latent part")
+    assert q.dtype == cache.dtype == out.dtype and q.is_contiguous() and out.is_contiguous() and cache.is_cuda
+    assert tiles.numel() >= 4 * n_rows and q.shape[-1] == H * dim and out.shape[-1] == H * vdim and (sink is None or sink.numel() >= H)
+    assert gate is None or (gate.dtype == q.dtype and ldg >= H)
+    assert n_splits <= 1 or (part is not None and part.numel() >= attn_softmax_part(out.shape[0], H, n_splits, vdim))
+    a = AttnLatentArgs(C.sizeof(AttnLatentArgs), _code(q), _p(q), q.shape[-1], _p(tiles), n_rows, _p(cache), slot_stride, row_stride, H, dim, vdim,
+                       float(scale), int(window), _p(sink), _p(gate), ldg, _p(out), out.shape[-1], n_splits, _p(part))
+    check(load().pcb_attn_latent(C.byref(a), _stream()), "pcb_attn_latent")

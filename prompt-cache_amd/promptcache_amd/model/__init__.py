@@ -23,7 +23,7 @@ import torch
 
 from ..pml import Preprocessor, PreprocessorList, escape_xml  # noqa: F401  (re-exported like the reference)
 from .config import (FALCON_SHAPES, MPT_SHAPES, SHAPES, BepepelShape, DibizenShape, FalconShape, FivesunShape, KazolornShape, LlamaShape, MptShape,
-                     architecture_of)
+                     PikadraShape, architecture_of)
 from .tokenizer import StandInTokenizer
 
 # HF hub ids the reference's drivers use (demo.py:27, eval.py:36, config/*.json) -> shape presets
@@ -444,8 +444,45 @@ class Bepepel(LanguageModel):
         return [t % self.config.vocab_size for t in super().encode(text)]
 
 
+class Pikadra(LanguageModel):
+    """Adapter of the Pikadra design (``config.PikadraShape``, ``pikadra_hip.PikadraHIP``).  A checkpoint directory holds
+    ``config.json`` and ``model.safetensors``; without one, ``shape=`` plus ``random_init=True`` (or ``weights=``) gives seeded
+    random weights.  ``dtype``: ``torch.bfloat16`` (serving) or ``torch.float32`` (everything in true 32-bit)."""
+
+    def __init__(self, name: Optional[str] = None, device: str = "cuda:0", shape: Optional[PikadraShape] = None,
+                 weights=None, tokenizer=None, random_init: bool = False, seed: int = 0, dtype=torch.bfloat16, **_kwargs):
+        from .pikadra_hip import PikadraHIP
+        from . import weights as W
+
+        if weights is not None:
+            assert shape is not None, "pass shape= together with weights="
+        elif name is not None and os.path.isdir(name):
+            shape = shape or PikadraShape.from_dir(name)
+            weights = W.load_pikadra_safetensors(name, shape)
+        else:
+            if shape is None or not random_init:
+                raise FileNotFoundError(f"no checkpoint directory {name!r}: pass one, or shape= with random_init=True")
+            weights = W.make_pikadra_weights(shape, seed, device=device)
+        if tokenizer is None:
+            tokenizer = StandInTokenizer(max(shape.vocab_size, 512))
+        model = PikadraHIP(shape, weights, device=device, dtype=dtype)
+        self.formatter = FormatConversation(system=("", "\n\n", ""), user=("User: ", "\n\nAssistant:"), assistant=(" ", "\n\n"))
+        super().__init__(name or shape.name, model, tokenizer, [tokenizer.eos_token_id], [])
+
+    def get_formatter(self) -> Callable[[str], str]:
+        return self.formatter
+
+    def get_cache_shape(self) -> Tuple[int, int, int]:
+        """(layer runs, 1, columns of a cached row) of the first layer: one latent row per token and run, whatever the head count."""
+        l = self.config.layers[0]
+        return len(self.config.runs()), 1, l.kv_rank + l.rot_dim
+
+    def encode(self, text: str) -> List[int]:
+        return [t % self.config.vocab_size for t in super().encode(text)]
+
+
 ADAPTERS = {"llama": Llama2, "falcon": Falcon, "mpt": Mpt, "kazolorn": Kazolorn, "dibizen": Dibizen, "fivesun": Fivesun,
-            "bepepel": Bepepel}
+            "bepepel": Bepepel, "pikadra": Pikadra}
 
 
 def load_language_model(path: str, **kwargs) -> LanguageModel:

@@ -1,10 +1,11 @@
-"""What the flat-row models share (``kazolorn_hip.KazolornHIP``, ``dibizen_hip.DibizenHIP``): requests live on slots of a
+"""What the flat-row models share (``kazolorn_hip.KazolornHIP``, ``dibizen_hip.DibizenHIP`` and those after them): requests live on slots of a
 ``SlotArena``, a step is ``forward_rows(arena, slots, tokens, want)`` over the new tokens of all its requests one after another,
 and the adapters' ``model(input_ids, past_key_values=...)`` convention is served on top of that."""
 from __future__ import annotations
 
 from typing import List, Optional
 
+import numpy as np
 import torch
 
 from .kv_arena import SlotArena
@@ -27,6 +28,34 @@ class SlotKV:
                     self.arena.free(s)
         except Exception:
             pass
+
+
+class StepRows:
+    """The flat rows of one step, laid out on the host and checked: ``counts`` / ``starts`` per request, ``row0`` each request's first
+    flat row, ``ids`` / ``row_slot`` / ``row_pos`` per row, ``want_rows`` the flat rows whose logits are asked for."""
+
+    def __init__(self, arena: SlotArena, slots, tokens, want, vocab: int):
+        counts = [len(t) for t in tokens]
+        if len(set(slots)) != len(slots) or len(slots) != len(tokens):
+            raise ValueError("one distinct slot per request")
+        if counts and min(counts) < 1:
+            raise ValueError("every request of a step brings at least one token")
+        self.counts, self.T, self.R = counts, sum(counts), len(counts)
+        self.want = [[c - 1] for c in counts] if want is None else want
+        self.ids = np.fromiter((t for req in tokens for t in req), dtype=np.int32, count=self.T)
+        if self.T and (self.ids.min() < 0 or self.ids.max() >= vocab):
+            raise ValueError("token id outside the vocabulary")
+        for b, ws in enumerate(self.want):
+            if any(not 0 <= int(w) < counts[b] for w in ws):
+                raise ValueError("a wanted place lies outside its request's tokens")
+        for s, c in zip(slots, counts):
+            arena.room_for(s, c)
+        self.starts = [arena.lengths[s] for s in slots]
+        self.row0 = np.concatenate([[0], np.cumsum(counts)]).astype(np.int64)
+        self.row_slot = np.repeat(np.asarray(slots, dtype=np.int64), counts)
+        self.row_pos = (np.concatenate([np.arange(c, dtype=np.int64) for c in counts]) if counts else np.zeros(0, np.int64)) + \
+            np.repeat(np.asarray(self.starts, dtype=np.int64), counts)
+        self.want_rows = np.asarray([int(self.row0[b]) + int(w) for b, ws in enumerate(self.want) for w in ws], dtype=np.int32)
 
 
 class SlotModel:
