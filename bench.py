@@ -824,6 +824,44 @@ def run_bepepel(args):
     print(json.dumps(out))
 
 
+def run_pikadra(args):
+    """Throughput of the Pikadra stack beside the Fivesun stack's latent attention (the closest existing model: the same
+    building-block library, bf16 tensors, an fp32 residual, one cached latent per token) at equal width, heads, head sizes and depth.
+
+    Per size: one prompt of 2048 tokens (tokens/s of the prefill), then decoding at a context of 2048 with 1 and 8 requests.
+    `dense` = the latent sizes (192 + 64 columns), the mask (none) and the feed-forward (a dense gated unit of 2 x width) of the Fivesun
+    stack; `moe` = 2 of 16 experts of width / 2 plus a shared one instead; `wide` = `dense` with a latent of 512 + 64 columns;
+    `loop` = `moe` with the middle two layers run twice (six layer runs).  Queries go through a latent of 3/8 of the width.  Random
+    weights, synthetic tokens."""
+    import torch
+    import __graft_entry__ as ge
+    ge.build()
+    from promptcache_amd.model import Fivesun, Pikadra
+    from promptcache_amd.model.config import FivesunShape, PikadraShape
+    dev = "cuda:0"
+    torch.cuda.set_device(0)
+    sizes = {"2k": dict(width=2048, heads=16), "4k": dict(width=4096, heads=32)}
+    L, V, T, steps, warm = 4, 32000, 2048, max(4, min(args.steps, 20)), max(1, min(args.warmup, 3))
+    g = torch.Generator().manual_seed(0)
+    out = {"metric": "pikadra_throughput", "unit": "tokens/s", "dtype": "bf16", "data": "synthetic", "layers": L, "prompt": T, "sizes": {}}
+    for key in args.pikadra_sizes.split(","):
+        c = sizes[key]
+        w, h = c["width"], c["heads"]
+        row = {"width": w, "heads": h}
+        if args.pikadra_baseline:
+            fs = FivesunShape.uniform(V, w, ["latent_attention"] * L, h, 1, w // h, 2 * w, window=0, kv_rank=192, rot_dim=64,
+                                      name=f"fivesun-{key}-latent")
+            row["fivesun_latent"] = slot_model_case(Fivesun(shape=fs, random_init=True, seed=0, device=dev), V, T, steps, warm, g)
+        for pk in args.pikadra_patterns.split(","):
+            ff = dict(dense_ff=2 * w) if pk in ("dense", "wide") else dict(experts=16, top=2, expert_ff=w // 2, shared_ff=w // 2)
+            shape = PikadraShape.uniform(V, w, L, h, w // h, 64, 512 if pk == "wide" else 192, 3 * w // 8,
+                                         loop=(1, 3, 2) if pk == "loop" else None, name=f"pikadra-{key}-{pk}", **ff)
+            row["pikadra_" + pk] = slot_model_case(Pikadra(shape=shape, random_init=True, seed=0, device=dev), V, T, steps, warm, g)
+        out["sizes"][key] = row
+        print(json.dumps({key: row}), file=sys.stderr, flush=True)
+    print(json.dumps(out))
+
+
 def run_kazolorn(args):
     """Throughput of the Kazolorn stack beside the MPT stack at equal width, heads, depth and feed-forward width.
 
@@ -927,6 +965,12 @@ def main():
                          "real models (random weights), beside the Kazolorn stack (the closest existing model) at equal size")
     ap.add_argument("--dibizen-sizes", default="2k,4k", help="--dibizen: which sizes (2k, 4k)")
     ap.add_argument("--dibizen-patterns", default="mixed,attention,lightning,mamba1", help="--dibizen: which layer patterns")
+    ap.add_argument("--pikadra", action="store_true",
+                    help="instead of the default workload: prefill / decode throughput of the Pikadra design at layer sizes of "
+                         "real models, beside the Fivesun stack's latent attention at equal size")
+    ap.add_argument("--pikadra-sizes", default="2k,4k", help="--pikadra: which sizes (2k, 4k)")
+    ap.add_argument("--pikadra-patterns", default="dense,moe,wide,loop", help="--pikadra: which stacks")
+    ap.add_argument("--pikadra-baseline", type=int, default=1, help="--pikadra: 0 leaves the Fivesun stack out (kernel profiles of Pikadra alone)")
     ap.add_argument("--bepepel", action="store_true",
                     help="instead of the default workload: prefill / decode throughput of the Bepepel design at layer sizes of "
                          "real models, beside the Dibizen stack at equal size")
@@ -948,6 +992,9 @@ def main():
         return
     if args.dibizen:
         run_dibizen(args)
+        return
+    if args.pikadra:
+        run_pikadra(args)
         return
     if args.bepepel:
         run_bepepel(args)

@@ -20,8 +20,8 @@ template <typename E, int KSQ, int VBW, int BK>
 __global__ __launch_bounds__(64 * LW) void attn_latent_kernel(pcb_attn_latent_args a) {
     constexpr int CE = 16 / sizeof(E);
     constexpr int KC = KSQ * 32, LD = v_ld<E>(KC), NKT = BK / 16, NK2 = BK / 32;
-    constexpr int NCH = BK * (KC / CE) / (64 * LW);
-    static_assert(BK * (KC / CE) % (64 * LW) == 0, "whole chunks per thread");
+    constexpr int LPR = 64 * LW / BK, NCH = KC / CE / LPR;           // threads that share a row: thread t loads row t / LPR, chunks t % LPR + i LPR
+    static_assert(KC / CE % LPR == 0, "whole chunks per thread");
     __shared__ __attribute__((aligned(16))) E Ks[BK * LD];
     __shared__ f4 Ss[NKT][64];                                       // scores of key tile kt as the result tile's lanes hold them
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, g = lane >> 4, c = lane & 15;
@@ -46,26 +46,30 @@ __global__ __launch_bounds__(64 * LW) void attn_latent_kernel(pcb_attn_latent_ar
         kb_hi = kb_lo + per - 1 < kb_hi ? kb_lo + per - 1 : kb_hi;
     }
     u32x4 rk[NCH];
+    const int lr = tid / LPR, lc = tid % LPR * CE;                   // this thread's row and first column
     auto fetch = [&](int kb) {
+        int j = kb * BK + lr;
+        j = j > pos ? pos : j;                                       // (keys past the end repeat the last one: finite, and masked)
+        const E* p = K + (int64_t)j * a.row_stride;
+        if (kvec) {
 #pragma unroll
-        for (int i = 0; i < NCH; ++i) {
-            const int t = tid + 64 * LW * i, r = t / (KC / CE), col = (t % (KC / CE)) * CE;
-            int j = kb * BK + r;
-            j = j > pos ? pos : j;                                   // (keys past the end repeat the last one: finite, and masked)
-            const E* p = K + (int64_t)j * a.row_stride;
-            u32x4 v = u32x4{0u, 0u, 0u, 0u};
-            if (kvec && col + CE <= dim) {
-                v = *reinterpret_cast<const u32x4*>(p + col);
-            } else if (col < dim) {
+            for (int i = 0; i < NCH; ++i) {
+                const int col = lc + i * LPR * CE;
+                rk[i] = u32x4{0u, 0u, 0u, 0u};
+                if (col < dim) rk[i] = *reinterpret_cast<const u32x4*>(p + col);
+            }
+        } else {
+#pragma unroll 1
+            for (int i = 0; i < NCH; ++i) {
+                const int col = lc + i * LPR * CE;
                 __attribute__((aligned(16))) E tmp[CE];
 #pragma unroll
                 for (int e = 0; e < CE; ++e) tmp[e] = col + e < dim ? p[col + e] : from_f32<E>(0.0f);
-                v = *reinterpret_cast<u32x4*>(tmp);
+                *reinterpret_cast<u32x4*>(&Ks[lr * LD + col]) = *reinterpret_cast<u32x4*>(tmp);
             }
-            rk[i] = v;
         }
     };
-    if (kb_lo <= kb_hi) fetch(kb_lo);
+    if (kvec && kb_lo <= kb_hi) fetch(kb_lo);
     Frag<E> qf[KSQ];
     const E* qp = (const E*)a.q + qrow * a.ldq + (int64_t)h * dim;
 #pragma unroll
@@ -77,13 +81,14 @@ __global__ __launch_bounds__(64 * LW) void attn_latent_kernel(pcb_attn_latent_ar
     for (int vb = 0; vb < VBW; ++vb) o[vb] = f4{0.f, 0.f, 0.f, 0.f};
     for (int kb = kb_lo; kb <= kb_hi; ++kb) {
         __syncthreads();                                             // the previous block's reads are done
+        if (kvec) {
 #pragma unroll
-        for (int i = 0; i < NCH; ++i) {
-            const int t = tid + 64 * LW * i;
-            *reinterpret_cast<u32x4*>(&Ks[t / (KC / CE) * LD + t % (KC / CE) * CE]) = rk[i];
+            for (int i = 0; i < NCH; ++i) *reinterpret_cast<u32x4*>(&Ks[lr * LD + lc + i * LPR * CE]) = rk[i];
+        } else {
+            fetch(kb);                                               // (odd sizes: element by element, straight into LDS)
         }
         __syncthreads();
-        if (kb < kb_hi) fetch(kb + 1);
+        if (kvec && kb < kb_hi) fetch(kb + 1);
         for (int kt = wave; kt < NKT; kt += LW) {
             f4 acc = f4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll

@@ -19,9 +19,8 @@ constexpr int PW = 4;          // waves of a workgroup
 
 // one 16-byte chunk of E starting at column c of a row whose columns [c_lo, c_hi) lie at p; others read as zero
 template <typename E>
-__device__ __forceinline__ u32x4 part_chunk(const E* p, int c, int c_lo, int c_hi, bool vec) {
+__device__ __forceinline__ u32x4 part_chunk(const E* p, int c, int c_lo, int c_hi) {
     constexpr int CE = 16 / sizeof(E);
-    if (vec && c >= c_lo && c + CE <= c_hi) return *reinterpret_cast<const u32x4*>(p + (c - c_lo));
     __attribute__((aligned(16))) E tmp[CE];
 #pragma unroll
     for (int e = 0; e < CE; ++e) tmp[e] = (c + e >= c_lo && c + e < c_hi) ? p[c + e - c_lo] : from_f32<E>(0.0f);
@@ -34,8 +33,9 @@ __global__ __launch_bounds__(64 * PW) void attn_prompt_kernel(pcb_attn_prompt_ar
     constexpr int CE = 16 / sizeof(E);
     constexpr int KC = KSQ * 32, VC = VB * 16;                       // columns of the tiles
     constexpr int KLD = KC + CE, VLD = v_ld<E>(VC);
-    constexpr int KCH = BK * (KC / CE) / (64 * PW), VCH = BK * (VC / CE) / (64 * PW);   // 16-byte chunks per thread
-    static_assert(BK * (KC / CE) % (64 * PW) == 0 && BK * (VC / CE) % (64 * PW) == 0, "whole chunks per thread");
+    constexpr int LPR = 64 * PW / BK;                                // threads that share a row: thread t loads row t / LPR, chunks t % LPR + i LPR
+    constexpr int KCH = KC / CE / LPR, VCH = VC / CE / LPR;          // 16-byte chunks per thread
+    static_assert(KC / CE % LPR == 0 && VC / CE % LPR == 0, "whole chunks per thread");
     constexpr int NKT = BK / 16, NK2 = BK / 32;
     __shared__ __attribute__((aligned(16))) E Ks[BK * KLD];
     __shared__ __attribute__((aligned(16))) E Vs[BK * VLD];
@@ -50,9 +50,10 @@ __global__ __launch_bounds__(64 * PW) void attn_prompt_kernel(pcb_attn_prompt_ar
     const E* V = (const E*)a.v + (int64_t)base * a.v_row_stride + (int64_t)hk * a.v_head_stride;
     const E* KT = (const E*)a.k_tail;
     const int32_t* trow = a.tail_rows ? a.tail_rows + base : nullptr;
-    const bool kvec = ((uintptr_t)a.k % 16 == 0) && a.k_row_stride % CE == 0 && a.k_head_stride % CE == 0;
-    const bool tvec = ((uintptr_t)a.k_tail % 16 == 0) && a.tail_row_stride % CE == 0 && split % CE == 0;
-    const bool vvec = ((uintptr_t)a.v % 16 == 0) && a.v_row_stride % CE == 0 && a.v_head_stride % CE == 0;
+    // whether every 16-byte chunk of a row lies in one part and can be read at once
+    const bool plain = ((uintptr_t)a.k % 16 == 0) && a.k_row_stride % CE == 0 && a.k_head_stride % CE == 0 && ((uintptr_t)a.v % 16 == 0) &&
+                       a.v_row_stride % CE == 0 && a.v_head_stride % CE == 0 && dim % CE == 0 && vdim % CE == 0 && split % CE == 0 &&
+                       (a.tail_dim == 0 || ((uintptr_t)a.k_tail % 16 == 0 && a.tail_row_stride % CE == 0));
 
     // this wave's queries
     const int w0 = wave * 16 * QT;                                   // first row of the wave within the tile
@@ -85,44 +86,52 @@ __global__ __launch_bounds__(64 * PW) void attn_prompt_kernel(pcb_attn_prompt_ar
     const int kb_lo = a.window > 0 && pos0 - a.window + 1 > 0 ? (pos0 - a.window + 1) / BK : 0;
     const int kb_hi = last / BK;
     u32x4 rk[KCH], rv[VCH];
+    const int lr = tid / LPR, lc = tid % LPR * CE;                   // this thread's row and first column
     auto fetch = [&](int kb) {
+        int j = kb * BK + lr;
+        j = j > last ? last : j;                                     // (keys past the end repeat the last one: finite, and masked)
+        const E* kp = K + (int64_t)j * a.k_row_stride;
+        const E* vp = V + (int64_t)j * a.v_row_stride;
+        const E* tp = a.tail_dim ? KT + (int64_t)(trow ? trow[j] : base + j) * a.tail_row_stride : kp;
+        if (plain) {
 #pragma unroll
-        for (int i = 0; i < KCH; ++i) {
-            const int t = tid + 64 * PW * i, r = t / (KC / CE), col = (t % (KC / CE)) * CE;
-            int j = kb * BK + r;
-            j = j > last ? last : j;                                 // (keys past the end repeat the last one: finite, and masked)
-            u32x4 v = u32x4{0u, 0u, 0u, 0u};
-            if (col < split) v = part_chunk<E>(K + (int64_t)j * a.k_row_stride, col, 0, split, kvec);
-            if (col + CE > split && col < dim) {
-                const E* tp = KT + (int64_t)(trow ? trow[j] : base + j) * a.tail_row_stride;
-                const u32x4 w = part_chunk<E>(tp, col, split, dim, tvec);
-                v = v | w;                                           // (the parts do not overlap, and what is not theirs is zero)
+            for (int i = 0; i < KCH; ++i) {
+                const int col = lc + i * LPR * CE;
+                rk[i] = u32x4{0u, 0u, 0u, 0u};
+                if (col < dim) rk[i] = *reinterpret_cast<const u32x4*>(col < split ? kp + col : tp + (col - split));
             }
-            rk[i] = v;
-        }
 #pragma unroll
-        for (int i = 0; i < VCH; ++i) {
-            const int t = tid + 64 * PW * i, r = t / (VC / CE), col = (t % (VC / CE)) * CE;
-            int j = kb * BK + r;
-            j = j > last ? last : j;
-            rv[i] = col < vdim ? part_chunk<E>(V + (int64_t)j * a.v_row_stride, col, 0, vdim, vvec) : u32x4{0u, 0u, 0u, 0u};
+            for (int i = 0; i < VCH; ++i) {
+                const int col = lc + i * LPR * CE;
+                rv[i] = u32x4{0u, 0u, 0u, 0u};
+                if (col < vdim) rv[i] = *reinterpret_cast<const u32x4*>(vp + col);
+            }
+        } else {
+#pragma unroll 1
+            for (int i = 0; i < KCH; ++i) {
+                const int col = lc + i * LPR * CE;
+                *reinterpret_cast<u32x4*>(&Ks[lr * KLD + col]) = part_chunk<E>(kp, col, 0, split) | part_chunk<E>(tp, col, split, dim);
+            }
+#pragma unroll 1
+            for (int i = 0; i < VCH; ++i) {
+                const int col = lc + i * LPR * CE;
+                *reinterpret_cast<u32x4*>(&Vs[lr * VLD + col]) = part_chunk<E>(vp, col, 0, vdim);
+            }
         }
     };
-    fetch(kb_lo);
+    if (plain) fetch(kb_lo);
     for (int kb = kb_lo; kb <= kb_hi; ++kb) {
         __syncthreads();                                             // the previous block's reads are done
+        if (plain) {
 #pragma unroll
-        for (int i = 0; i < KCH; ++i) {
-            const int t = tid + 64 * PW * i;
-            *reinterpret_cast<u32x4*>(&Ks[t / (KC / CE) * KLD + t % (KC / CE) * CE]) = rk[i];
-        }
+            for (int i = 0; i < KCH; ++i) *reinterpret_cast<u32x4*>(&Ks[lr * KLD + lc + i * LPR * CE]) = rk[i];
 #pragma unroll
-        for (int i = 0; i < VCH; ++i) {
-            const int t = tid + 64 * PW * i;
-            *reinterpret_cast<u32x4*>(&Vs[t / (VC / CE) * VLD + t % (VC / CE) * CE]) = rv[i];
+            for (int i = 0; i < VCH; ++i) *reinterpret_cast<u32x4*>(&Vs[lr * VLD + lc + i * LPR * CE]) = rv[i];
+        } else {
+            fetch(kb);                                               // (odd sizes: element by element, straight into LDS)
         }
         __syncthreads();
-        if (kb < kb_hi) fetch(kb + 1);
+        if (plain && kb < kb_hi) fetch(kb + 1);
         const int k0 = kb * BK;
         if (!busy || k0 > w_last || (a.window > 0 && k0 + BK - 1 < w_first - a.window + 1)) continue;
 
