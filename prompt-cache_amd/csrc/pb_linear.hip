@@ -5,6 +5,7 @@
 // Tiling: workgroup = 4 waves in a 2 x 2 grid, a wave owns TM x TN result tiles of 16 x 16, so the workgroup covers
 // (32 TM) x (32 TN) of Y.  Per stage of two 32-element k-steps the A and B panels go global -> registers -> LDS (the next stage's
 // loads are in flight while this stage's MFMAs run); waves read their operand fragments from LDS with one 16-byte read per fragment (bf16).
+// bf16 operands that can be read in 16-byte chunks take linear_dma_kernel below instead; fp32, odd sizes and scaled rows this one.
 #include "pb_common.h"
 
 namespace {
@@ -59,6 +60,14 @@ __device__ __forceinline__ float apply_act(int act, float v, float param) {
     }
 }
 
+// the gated epilogue's function: silu (the default), relu or the tanh-form gelu, which is z sigmoid(2 u) for tanh's argument u.  Kept short:
+// an epilogue too long to unroll would index the accumulators, which throws them out of the registers.
+__device__ __forceinline__ float gate_act(int act, float v) {
+    const float t = act == PCB_ACT_GELU_TANH ? 1.5957691216057308f * (v + 0.044715f * v * v * v) : v;
+    const float s = v / (1.0f + expf(-t));
+    return act == PCB_ACT_RELU ? fmaxf(v, 0.0f) : s;
+}
+
 // one result element through the epilogue (see pcb_linear_args)
 template <typename E, int EPI>
 __device__ __forceinline__ void emit(const pcb_linear_args& a, int m, int n, float acc, float acc2, float bv, float cs, float bv2 = 0.0f) {
@@ -67,7 +76,7 @@ __device__ __forceinline__ void emit(const pcb_linear_args& a, int m, int n, flo
         // (the split-off parts are stored as they are)
         v = apply_act((a.act_split > 0 && n >= a.act_split) ? a.act2 : a.act, v, a.act_param);
     if (EPI == PCB_EPI_SILU_MUL) {
-        v = apply_act(a.act == PCB_ACT_NONE ? PCB_ACT_SILU : a.act, v, 0.0f) * (acc2 + bv2);
+        v = gate_act(a.act, v) * (acc2 + bv2);
         if (a.row_gate) v *= to_f32(((const E*)a.row_gate)[m * a.ld_row_gate]);
     }
     if (EPI == PCB_EPI_SCALE_ADD) {
@@ -336,6 +345,172 @@ __global__ __launch_bounds__(64 * SKW) void linear_skinny_kernel(pcb_linear_args
     }
 }
 
+// ---- many rows in bf16: both panels travel to LDS by themselves --------------------------------------------------------------------
+// The same tiles (2 x 2 waves of TM x TN result tiles) for operands whose rows can be read in 16-byte chunks: global_load_lds carries a
+// stage of 64 k elements (1 KiB per wave instruction: 8 rows x 128 bytes) straight into a double-buffered image, one barrier per stage, so
+// no register and no branch stands between the loads.  Rows past the end repeat the last one (their results are not stored); chunks
+// past K come from a block of zeros.  The 16-byte chunk c of row r sits at position c ^ ((r >> 1) & 7) of its 128-byte row, which spreads
+// a fragment read over all banks; the loads write lane by lane, so the permutation is applied to each lane's source.
+// A plain launch numbers its tiles panel by panel (all row blocks of a column panel in turn) and gives each XCD one run of them: a
+// panel's weights are fetched into one L2.
+__device__ const u32x4 zero_row = {0u, 0u, 0u, 0u};
+
+__device__ __forceinline__ void dma16(const void* g, void* lds_wave_base) {
+    __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)g, (__attribute__((address_space(3))) void*)lds_wave_base, 16,
+                                     0, 0);
+}
+
+template <int EPI, int TM, int TN>
+__global__ __launch_bounds__(256) void linear_dma_kernel(pcb_linear_args a) {
+    typedef bf16_t E;
+    constexpr bool TWO = EPI == PCB_EPI_SILU_MUL;
+    constexpr int BM = 32 * TM, BN = 32 * TN, ROWS = BM + (TWO ? 2 : 1) * BN, BK = 64;
+    constexpr int NI = ROWS / 32;                                    // wave instructions per wave and stage
+    __shared__ __attribute__((aligned(16))) E img[2][ROWS * BK];
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+    const int wm = wave >> 1, wn = wave & 1, group = lane >> 4, l15 = lane & 15;
+    const int K = a.K, N = a.N;
+
+    int g = 0, m_lo = -1, m_hi = 0, n_lo;
+    if (a.n_groups > 0) {
+        int t = blockIdx.y;
+        for (g = 0; g < a.n_groups; ++g) {
+            const int lo = a.group_off[g], hi = a.group_off[g + 1];
+            const int nt = (hi - lo + BM - 1) / BM;
+            if (t < nt) {
+                m_lo = lo + t * BM;
+                m_hi = hi;
+                break;
+            }
+            t -= nt;
+        }
+        if (m_lo < 0) return;
+        n_lo = blockIdx.x * BN;
+    } else {
+        const int mb = (a.M + BM - 1) / BM, total = mb * ((N + BN - 1) / BN), per = (total + 7) / 8;
+        const int t = (blockIdx.x & 7) * per + (blockIdx.x >> 3);
+        if ((int)(blockIdx.x >> 3) >= per || t >= total) return;
+        m_lo = t % mb * BM;
+        m_hi = a.M;
+        n_lo = t / mb * BN;
+        if (a.n_batch > 0) g = blockIdx.z;
+    }
+    const E* W = (const E*)a.w + (int64_t)g * a.w_group_stride;
+    const E* W2 = TWO ? (const E*)a.w2 + (int64_t)g * a.w_group_stride : nullptr;
+    const E* X = (const E*)a.x + (a.n_batch > 0 ? (int64_t)blockIdx.z * a.x_batch_stride : 0);
+
+    // instruction i of this wave fills rows 8 (4 i + wave) .. + 7 of the image: A rows, then W rows, then W2 rows
+    const E* src[NI];
+    int kc[NI];                                                      // the lane's k offset within the stage
+#pragma unroll
+    for (int i = 0; i < NI; ++i) {
+        const int r = 8 * (4 * i + wave) + (lane >> 3);
+        kc[i] = ((lane & 7) ^ ((r >> 1) & 7)) * 8;
+        if (32 * i < BM) {
+            int m = m_lo + r;
+            m = m < m_hi ? m : m_hi - 1;
+            src[i] = X + (int64_t)(a.row_src ? a.row_src[m] : m) * a.ldx;
+        } else {
+            const bool second = TWO && 32 * i >= BM + BN;
+            int n = n_lo + r - BM - (second ? BN : 0);
+            n = n < N ? n : N - 1;
+            src[i] = (second ? W2 : W) + (int64_t)n * a.ldw;
+        }
+    }
+    auto fetch = [&](int k0, int buf) {
+        if (k0 + BK <= K) {
+#pragma unroll
+            for (int i = 0; i < NI; ++i) dma16(src[i] + k0 + kc[i], &img[buf][(4 * i + wave) * 8 * BK]);
+        } else {
+#pragma unroll
+            for (int i = 0; i < NI; ++i)
+                dma16(k0 + kc[i] < K ? (const void*)(src[i] + k0 + kc[i]) : (const void*)&zero_row, &img[buf][(4 * i + wave) * 8 * BK]);
+        }
+    };
+    f4 acc[TM][TN], acc2[TWO ? TM : 1][TWO ? TN : 1];
+#pragma unroll
+    for (int i = 0; i < TM; ++i)
+#pragma unroll
+        for (int j = 0; j < TN; ++j) {
+            acc[i][j] = f4{0.f, 0.f, 0.f, 0.f};
+            if (TWO) acc2[i][j] = f4{0.f, 0.f, 0.f, 0.f};
+        }
+    auto frag = [&](int buf, int r, int ks) {
+        Frag<E> f;
+        f.v = *reinterpret_cast<const u32x4*>(&img[buf][r * BK + ((4 * ks + group) ^ ((r >> 1) & 7)) * 8]);
+        return f;
+    };
+    fetch(0, 0);
+    int buf = 0;
+    for (int k0 = 0; k0 < K; k0 += BK, buf ^= 1) {
+        asm volatile("s_waitcnt vmcnt(0)" ::: "memory");             // this wave's part of the stage has landed
+        __syncthreads();                                             // so has everyone's, and the other buffer is read out
+        if (k0 + BK < K) fetch(k0 + BK, buf ^ 1);
+#pragma unroll
+        for (int ks = 0; ks < 2; ++ks) {
+            Frag<E> fa[TM];
+#pragma unroll
+            for (int i = 0; i < TM; ++i) fa[i] = frag(buf, (wm * TM + i) * 16 + l15, ks);
+#pragma unroll
+            for (int j = 0; j < TN; ++j) {
+                const Frag<E> fb = frag(buf, BM + (wn * TN + j) * 16 + l15, ks);
+#pragma unroll
+                for (int i = 0; i < TM; ++i) acc[i][j] = mma(fa[i], fb, acc[i][j]);
+                if (TWO) {
+                    const Frag<E> fb2 = frag(buf, BM + BN + (wn * TN + j) * 16 + l15, ks);
+#pragma unroll
+                    for (int i = 0; i < TM; ++i) acc2[i][j] = mma(fa[i], fb2, acc2[i][j]);
+                }
+            }
+        }
+    }
+
+    const E* bias = (const E*)a.bias;
+#pragma unroll
+    for (int j = 0; j < TN; ++j) {
+        const int n = n_lo + (wn * TN + j) * 16 + l15;
+        if (n >= N) continue;
+        const float bv = bias ? to_f32(bias[n]) : 0.0f;
+        const float bv2 = (TWO && a.bias2) ? to_f32(((const E*)a.bias2)[n]) : 0.0f;
+        const float cs = (EPI == PCB_EPI_SCALE_ADD) ? a.col_scale[n] : 0.0f;
+#pragma unroll
+        for (int i = 0; i < TM; ++i)
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+                const int m = m_lo + (wm * TM + i) * 16 + 4 * group + r;
+                if (m < m_hi) emit<E, EPI>(a, m, n, acc[i][j][r], TWO ? acc2[i][j][r] : 0.0f, bv, cs, bv2);
+            }
+    }
+}
+
+template <int EPI, int TM, int TN>
+int launch_dma(const pcb_linear_args& a, hipStream_t stream) {
+    constexpr int BM = 32 * TM, BN = 32 * TN;
+    const int nb = pcb_ceil_div(a.N, BN), mb = pcb_ceil_div(a.M, BM);
+    const dim3 grid = a.n_groups > 0 ? dim3(nb, mb + a.n_groups) : dim3(8 * pcb_ceil_div(nb * mb, 8), 1, a.n_batch > 0 ? a.n_batch : 1);
+    hipLaunchKernelGGL((linear_dma_kernel<EPI, TM, TN>), grid, dim3(256), 0, stream, a);
+    return pcb_check_launch("linear_dma_kernel");
+}
+
+// whether every operand row can be read in 16-byte chunks (bf16)
+bool dma_ok(const pcb_linear_args& a) {
+    return a.dtype == PCB_BF16 && !a.row_scale && a.K % 8 == 0 && a.ldx % 8 == 0 && a.ldw % 8 == 0 && a.w_group_stride % 8 == 0 &&
+           a.x_batch_stride % 8 == 0 && ((uintptr_t)a.x | (uintptr_t)a.w | (uintptr_t)a.w2) % 16 == 0 &&
+           (int64_t)pcb_ceil_div(a.N, 32) * pcb_ceil_div(a.M, 32) < (1 << 30);
+}
+
+template <int EPI>
+int dispatch_dma(const pcb_linear_args& a, int rows, hipStream_t stream) {
+    // the largest tile that still gives every CU a workgroup; grouped launches count the tiles their rows fill
+    constexpr int TNW = EPI == PCB_EPI_SILU_MUL ? 2 : 4;
+    const int64_t batch = a.n_batch > 0 ? a.n_batch : 1;
+    auto tiles = [&](int bm, int bn) { return batch * pcb_ceil_div(a.M, bm) * pcb_ceil_div(a.N, bn); };
+    if (rows > 64 && tiles(128, 32 * TNW) >= 256) return launch_dma<EPI, 4, TNW>(a, stream);
+    if (rows > 32 && tiles(64, 32 * TNW) >= 256) return launch_dma<EPI, 2, TNW>(a, stream);
+    if (rows > 32) return launch_dma<EPI, 2, TNW / 2>(a, stream);
+    return launch_dma<EPI, 1, TNW / 2>(a, stream);
+}
+
 template <typename E, int EPI, int TM, int TN>
 int launch(const pcb_linear_args& a, hipStream_t stream) {
     constexpr int BM = 32 * TM, BN = 32 * TN;
@@ -364,6 +539,13 @@ int dispatch(const pcb_linear_args& a, hipStream_t stream) {
                 hipLaunchKernelGGL((linear_skinny_kernel<E, PCB_EPI_SCALE_ADD>), grid, dim3(64 * SKW), 0, stream, a);
         }
         return pcb_check_launch("linear_skinny_kernel");
+    }
+    if (sizeof(E) == 2 && dma_ok(a)) {
+        switch (a.epilogue) {
+            case PCB_EPI_STORE: return dispatch_dma<PCB_EPI_STORE>(a, rows, stream);
+            case PCB_EPI_SILU_MUL: return dispatch_dma<PCB_EPI_SILU_MUL>(a, rows, stream);
+            default: return dispatch_dma<PCB_EPI_SCALE_ADD>(a, rows, stream);
+        }
     }
     switch (a.epilogue) {
         case PCB_EPI_STORE:
