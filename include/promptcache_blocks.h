@@ -590,7 +590,8 @@ int pcb_attn_prompt(const pcb_attn_prompt_args* a, void* stream);
 /* Causal softmax attention of single rows over one key head whose values are the first vdim columns of the dim-column key rows
  * themselves (decoding over a shared latent).  tile r = {slot, position, 1, flat row} (int32 x 4, device); key j of slot s: cache +
  * s * slot_stride + j * row_stride.  q: head h at column h * dim; out: head h at column h * vdim.  window, sink, gate (one number per row
- * and head), n_splits and part as in pcb_attn_softmax.  dim <= 768, vdim <= 512. */
+ * and head) and n_splits as in pcb_attn_softmax; part: fp32 scratch of n_rows * H * n_splits * (vdim + 2) floats.  dim <= 768,
+ * vdim <= 512. */
 typedef struct pcb_attn_latent_args {
     uint32_t struct_bytes;
     int32_t dtype;

@@ -143,8 +143,9 @@ __global__ __launch_bounds__(64 * LW) void attn_latent_kernel(pcb_attn_latent_ar
     float* pp = nullptr;
     E* op = nullptr;
     if (a.n_splits > 1) {
-        pp = a.part + ((qrow * a.H + h) * a.n_splits + blockIdx.z) * (int64_t)(vdim + 2);
-        if (wave == 0 && g == 0) pp[vdim] = m, pp[vdim + 1] = l;
+        const int64_t run = ((int64_t)blockIdx.x * a.H + h) * a.n_splits + blockIdx.z;
+        pp = a.part + run * vdim;
+        if (wave == 0 && g == 0) *reinterpret_cast<float2*>(a.part + (int64_t)a.n_rows * a.H * a.n_splits * vdim + 2 * run) = float2{m, l};
     } else {
         float keep = 1.0f;
         if (a.sink) {
@@ -157,18 +158,26 @@ __global__ __launch_bounds__(64 * LW) void attn_latent_kernel(pcb_attn_latent_ar
         if (a.gate) f *= to_f32(((const E*)a.gate)[qrow * a.ldg + h]);
         op = (E*)a.out + qrow * a.ldo + (int64_t)h * vdim;
     }
+    const bool quads = vdim % 4 == 0 && (pp || (((uintptr_t)a.out % 16 == 0) && a.ldo % 4 == 0));
 #pragma unroll
-    for (int vb = 0; vb < VBW; ++vb)
-#pragma unroll
-        for (int r = 0; r < 4; ++r) {
-            const int col = (wave * VBW + vb) * 16 + 4 * g + r;
-            if (col < vdim) {
-                if (pp)
-                    pp[col] = o[vb][r];
-                else
-                    op[col] = from_f32<E>(o[vb][r] * f);
-            }
+    for (int vb = 0; vb < VBW; ++vb) {
+        const int col = (wave * VBW + vb) * 16 + 4 * g;
+        if (quads && col < vdim) {
+            if (pp)
+                *reinterpret_cast<f4*>(pp + col) = o[vb];
+            else
+                store4(op + col, o[vb][0] * f, o[vb][1] * f, o[vb][2] * f, o[vb][3] * f);
+            continue;
         }
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+            if (col + r < vdim) {
+                if (pp)
+                    pp[col + r] = o[vb][r];
+                else
+                    op[col + r] = from_f32<E>(o[vb][r] * f);
+            }
+    }
 }
 
 // one workgroup per (row, head): the runs' factors once, then their partial results rescaled to the common maximum and summed
@@ -177,11 +186,13 @@ __global__ __launch_bounds__(256) void attn_latent_merge_kernel(pcb_attn_latent_
     __shared__ float fac[64];
     const int64_t qrow = a.tiles[4 * blockIdx.x + 3];
     const int h = blockIdx.y, vdim = a.vdim, Z = a.n_splits, lane = threadIdx.x & 63;
-    const float* pp = a.part + (qrow * a.H + h) * Z * (int64_t)(vdim + 2);
+    const int64_t run = ((int64_t)blockIdx.x * a.H + h) * Z;
+    const float* pp = a.part + run * vdim;
+    const float* ml = a.part + (int64_t)a.n_rows * a.H * Z * vdim + 2 * run;
     if (threadIdx.x < 64) {
         const float NEG = -__builtin_inff();
-        const float mz = lane < Z ? pp[(int64_t)lane * (vdim + 2) + vdim] : NEG;
-        const float lz = lane < Z ? pp[(int64_t)lane * (vdim + 2) + vdim + 1] : 0.0f;
+        const float mz = lane < Z ? ml[2 * lane] : NEG;
+        const float lz = lane < Z ? ml[2 * lane + 1] : 0.0f;
         float top = wave_max(mz);                                    // (the row sees itself: a number)
         const float sk = a.sink ? a.sink[h] * 1.44269504088896f : NEG;
         top = fmaxf(top, sk);
@@ -194,10 +205,8 @@ __global__ __launch_bounds__(256) void attn_latent_merge_kernel(pcb_attn_latent_
     __syncthreads();
     for (int c = threadIdx.x; c < vdim; c += 256) {
         float o = 0.0f;
-        for (int z = 0; z < Z; ++z) {
-            const float f = fac[z];
-            if (f != 0.0f) o += f * pp[(int64_t)z * (vdim + 2) + c];
-        }
+#pragma unroll 8
+        for (int z = 0; z < Z; ++z) o += fac[z] * pp[(int64_t)z * vdim + c];       // (an empty run left zeros)
         ((E*)a.out)[qrow * a.ldo + (int64_t)h * vdim + c] = from_f32<E>(o);
     }
 }
@@ -231,6 +240,7 @@ PCB_EXPORT int pcb_attn_latent(const pcb_attn_latent_args* a, void* stream) {
                 PCB_ERR_ARG, "pcb_attn_latent: bad sizes (rows of up to 768 columns, of which up to 512 are the value)");
     if (a->n_rows == 0) return PCB_OK;
     PCB_REQUIRE(a->q && a->tiles && a->cache && a->out && (!a->gate || a->ldg >= a->H), PCB_ERR_ARG, "pcb_attn_latent: null pointer");
-    PCB_REQUIRE(a->n_splits <= 1 || (a->part && a->n_splits <= 64), PCB_ERR_ARG, "pcb_attn_latent: up to 64 runs, with their scratch");
+    PCB_REQUIRE(a->n_splits <= 1 || (a->part && (uintptr_t)a->part % 16 == 0 && a->n_splits <= 64), PCB_ERR_ARG,
+                "pcb_attn_latent: up to 64 runs, with their scratch");
     return a->dtype == PCB_BF16 ? dispatch<pcb::bf16_t>(*a, (hipStream_t)stream) : dispatch<float>(*a, (hipStream_t)stream);
 }

@@ -14,34 +14,31 @@ using namespace pcb;
 
 constexpr int MAX_PAIRS = 512;   // rotated column pairs per head
 
-template <typename E>
-__global__ __launch_bounds__(256) void head_prep_kernel(pcb_head_prep_args a) {
-    __shared__ float cs[MAX_PAIRS], sn[MAX_PAIRS];
-    const pcb_head_prep_seg& s = a.seg[blockIdx.y];
-    const int64_t row = blockIdx.x;
-    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, waves = blockDim.x >> 6;
+// the heads of one segment for one row: a wave takes a head (lanes step through its pairs), or -- LONE, a segment of one head: a latent of
+// hundreds of columns -- the whole workgroup does
+template <typename E, bool LONE>
+__device__ __forceinline__ void prep_heads(const pcb_head_prep_args& a, const pcb_head_prep_seg& s, int64_t row, const float* cs, const float* sn,
+                                           float* red) {
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     const int D = s.head_dim, np = s.rot_dims / 2;
-    if (np > 0) {
-        const double p = (double)a.pos[row];
-        for (int i = threadIdx.x; i < np; i += blockDim.x) {
-            double sv, cv;
-            sincos(p * a.freqs[i], &sv, &cv);
-            cs[i] = (float)cv * a.rot_mag;
-            sn[i] = (float)sv * a.rot_mag;
-        }
-        __syncthreads();
-    }
+    const int first = LONE ? (int)threadIdx.x : lane;
+    constexpr int STEP = LONE ? 256 : 64;
     const float lam = s.blend ? s.blend[0] : 0.0f;
-    for (int h = wave; h < s.heads; h += waves) {
+    for (int h = LONE ? 0 : wave; h < s.heads; h += 4) {
         const E* x = (const E*)s.src + row * s.ld_src + (int64_t)h * s.src_head_stride;
         float inv = 1.0f;
         if (s.norm) {
             float ss = 0.0f;
-            for (int c = lane; c < D; c += 64) {
+            for (int c = first; c < D; c += STEP) {
                 const float v = to_f32(x[c]);
                 ss += v * v;
             }
             ss = wave_sum(ss);
+            if (LONE) {
+                if (lane == 0) red[wave] = ss;
+                __syncthreads();                             // (also: every column is read before one is written in place)
+                ss = red[0] + red[1] + red[2] + red[3];
+            }
             inv = 1.0f / sqrtf(ss / (float)D + a.eps);
         }
         const float* __restrict__ other = s.blend ? s.other + row * s.ld_other + (int64_t)h * D : nullptr;
@@ -49,7 +46,7 @@ __global__ __launch_bounds__(256) void head_prep_kernel(pcb_head_prep_args a) {
         E* dst = (E*)s.dst + (s.row_off ? s.row_off[row] : row * s.ld_dst) + (int64_t)h * s.head_stride;
         // a lane owns whole pairs: pair i < np turns by the position; of the columns that do not turn, pair i >= np is the next two
         // (interleaved rotation: the pairs in memory order, np of them from rot_off on)
-        for (int i0 = lane; 2 * i0 < D + 1; i0 += 64) {
+        for (int i0 = first; 2 * i0 < D + 1; i0 += STEP) {
             int c[2];
             int i = -1;                                      // which angle, or none
             if (a.rot_half && np > 0) {
@@ -92,6 +89,28 @@ __global__ __launch_bounds__(256) void head_prep_kernel(pcb_head_prep_args a) {
                 if (c[e] < D) dst[(int64_t)c[e] * s.col_stride] = from_f32<E>(v[e]);
         }
     }
+}
+
+template <typename E>
+__global__ __launch_bounds__(256) void head_prep_kernel(pcb_head_prep_args a) {
+    __shared__ float cs[MAX_PAIRS], sn[MAX_PAIRS], red[4];
+    const pcb_head_prep_seg& s = a.seg[blockIdx.y];
+    const int64_t row = blockIdx.x;
+    const int np = s.rot_dims / 2;
+    if (np > 0) {
+        const double p = (double)a.pos[row];
+        for (int i = threadIdx.x; i < np; i += 256) {
+            double sv, cv;
+            sincos(p * a.freqs[i], &sv, &cv);
+            cs[i] = (float)cv * a.rot_mag;
+            sn[i] = (float)sv * a.rot_mag;
+        }
+        __syncthreads();
+    }
+    if (s.heads == 1)
+        prep_heads<E, true>(a, s, row, cs, sn, red);
+    else
+        prep_heads<E, false>(a, s, row, cs, sn, red);
 }
 
 }  // namespace

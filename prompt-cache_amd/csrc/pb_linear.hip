@@ -6,6 +6,8 @@
 // (32 TM) x (32 TN) of Y.  Per stage of two 32-element k-steps the A and B panels go global -> registers -> LDS (the next stage's
 // loads are in flight while this stage's MFMAs run); waves read their operand fragments from LDS with one 16-byte read per fragment (bf16).
 // bf16 operands that can be read in 16-byte chunks take linear_dma_kernel below instead; fp32, odd sizes and scaled rows this one.
+#include <type_traits>
+
 #include "pb_common.h"
 
 namespace {
@@ -68,17 +70,9 @@ __device__ __forceinline__ float gate_act(int act, float v) {
     return act == PCB_ACT_RELU ? fmaxf(v, 0.0f) : s;
 }
 
-// one result element through the epilogue (see pcb_linear_args)
+// where one finished element goes (see pcb_linear_args)
 template <typename E, int EPI>
-__device__ __forceinline__ void emit(const pcb_linear_args& a, int m, int n, float acc, float acc2, float bv, float cs, float bv2 = 0.0f) {
-    float v = acc + bv;
-    if (EPI == PCB_EPI_STORE && (a.act | a.act2) && !(a.split_n > 0 && n >= a.split_n) && !(a.split_n3 > 0 && n >= a.split_n3))
-        // (the split-off parts are stored as they are)
-        v = apply_act((a.act_split > 0 && n >= a.act_split) ? a.act2 : a.act, v, a.act_param);
-    if (EPI == PCB_EPI_SILU_MUL) {
-        v = gate_act(a.act, v) * (acc2 + bv2);
-        if (a.row_gate) v *= to_f32(((const E*)a.row_gate)[m * a.ld_row_gate]);
-    }
+__device__ __forceinline__ void put(const pcb_linear_args& a, int m, int n, float v, float cs) {
     if (EPI == PCB_EPI_SCALE_ADD) {
         float* y = (float*)a.y + (int64_t)m * a.ldy + n;
         const float b0 = a.base ? a.base[(int64_t)m * a.ldbase + n] : *y;
@@ -104,6 +98,24 @@ __device__ __forceinline__ void emit(const pcb_linear_args& a, int m, int n, flo
         ((float*)a.y)[at] = v;
     else
         ((E*)a.y)[at] = from_f32<E>(v);
+}
+
+// columns that pass through act / act2 of a plain store: the split-off parts are stored as they are
+__device__ __forceinline__ int act_end(const pcb_linear_args& a) {
+    return a.split_n > 0 ? a.split_n : (a.split_n3 > 0 ? a.split_n3 : a.N);
+}
+
+// one result element through the epilogue
+template <typename E, int EPI>
+__device__ __forceinline__ void emit(const pcb_linear_args& a, int m, int n, float acc, float acc2, float bv, float cs, float bv2 = 0.0f) {
+    float v = acc + bv;
+    if (EPI == PCB_EPI_STORE && (a.act | a.act2) && n < act_end(a))
+        v = apply_act((a.act_split > 0 && n >= a.act_split) ? a.act2 : a.act, v, a.act_param);
+    if (EPI == PCB_EPI_SILU_MUL) {
+        v = gate_act(a.act, v) * (acc2 + bv2);
+        if (a.row_gate) v *= to_f32(((const E*)a.row_gate)[m * a.ld_row_gate]);
+    }
+    put<E, EPI>(a, m, n, v, cs);
 }
 
 template <typename E, int EPI, int TM, int TN>
@@ -245,7 +257,7 @@ __global__ __launch_bounds__(256) void linear_kernel(pcb_linear_args a) {
 }
 
 // ---- few rows: the weights stream once, straight from memory into the matrix cores --------------------------------------------
-// Workgroup = 16 result columns x up to 16 rows; its eight waves split the k range (k-step s goes to wave s % 8) and add their
+// Workgroup = 16 result columns x up to 16 rows; its SKW waves split the k range (k-step s goes to wave s % SKW) and add their
 // partial tiles through LDS.  No LDS staging: a lane's B fragment is 16 contiguous bytes of its weight row, its A fragment 16
 // bytes of its activation row (a handful of rows that stay in cache).
 template <typename E>
@@ -265,9 +277,21 @@ __device__ __forceinline__ void scale_frag<float>(Frag<float>& f, float s) {
     for (int e = 0; e < 8; ++e) f.v[e] *= s;
 }
 
-constexpr int SKW = 8;          // waves of a few-row workgroup
+// the lane's elements of a whole k-step; p points at the first of them
+__device__ __forceinline__ Frag<bf16_t> whole_frag(const bf16_t* p) {
+    Frag<bf16_t> f;
+    f.v = *reinterpret_cast<const u32x4*>(p);
+    return f;
+}
+__device__ __forceinline__ Frag<float> whole_frag(const float* p) {
+    Frag<float> f;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) f.v[e] = p[4 * e];
+    return f;
+}
 
-template <typename E, int EPI>
+// SKW: waves of a workgroup (eight, or sixteen where few workgroups walk a long k range)
+template <typename E, int EPI, int SKW>
 __global__ __launch_bounds__(64 * SKW) void linear_skinny_kernel(pcb_linear_args a) {
     constexpr bool TWO = EPI == PCB_EPI_SILU_MUL;
     constexpr int CE = Tile<E>::CE;
@@ -309,8 +333,23 @@ __global__ __launch_bounds__(64 * SKW) void linear_skinny_kernel(pcb_linear_args
     const float xs = (scaled && a_ok) ? a.row_scale[m_a] : 1.0f;
     f4 acc = f4{0.f, 0.f, 0.f, 0.f}, acc2 = f4{0.f, 0.f, 0.f, 0.f};
     const int nsteps = (K + 31) / 32;
+    // whole k-steps of rows that can be read in 16-byte pieces: nothing between the loads.  (Lanes past the last row or column read row 0
+    // or column 0 instead: what they multiply is not stored.)
+    int st = wave;
+    if (vec && !scaled) {
+        const int whole = K / 32;
+        const E* xp = xrow + (sizeof(E) == 2 ? 8 * group : group);
+        const E* wp = wrow + (sizeof(E) == 2 ? 8 * group : group);
+        const E* wp2 = TWO ? wrow2 + (sizeof(E) == 2 ? 8 * group : group) : nullptr;
 #pragma unroll 8
-    for (int st = wave; st < nsteps; st += SKW) {
+        for (; st < whole; st += SKW) {
+            const Frag<E> fa = whole_frag(xp + 32 * st), fb = whole_frag(wp + 32 * st);
+            acc = mma(fa, fb, acc);
+            if (TWO) acc2 = mma(fa, whole_frag(wp2 + 32 * st), acc2);
+        }
+    }
+#pragma unroll 2
+    for (; st < nsteps; st += SKW) {
         const int k0 = 32 * st;
         Frag<E> fa = load_frag(xrow + k0, group, a_ok ? K - k0 : 0, vec);
         if (scaled) scale_frag<E>(fa, xs);
@@ -347,7 +386,7 @@ __global__ __launch_bounds__(64 * SKW) void linear_skinny_kernel(pcb_linear_args
 
 // ---- many rows in bf16: both panels travel to LDS by themselves --------------------------------------------------------------------
 // The same tiles (2 x 2 waves of TM x TN result tiles) for operands whose rows can be read in 16-byte chunks: global_load_lds carries a
-// stage of 64 k elements (1 KiB per wave instruction: 8 rows x 128 bytes) straight into a double-buffered image, one barrier per stage, so
+// stage of 64 k elements (1 KiB per wave instruction: 8 rows x 128 bytes) straight into a ring of two or three images, one barrier per stage, so
 // no register and no branch stands between the loads.  Rows past the end repeat the last one (their results are not stored); chunks
 // past K come from a block of zeros.  The 16-byte chunk c of row r sits at position c ^ ((r >> 1) & 7) of its 128-byte row, which spreads
 // a fragment read over all banks; the loads write lane by lane, so the permutation is applied to each lane's source.
@@ -360,13 +399,13 @@ __device__ __forceinline__ void dma16(const void* g, void* lds_wave_base) {
                                      0, 0);
 }
 
-template <int EPI, int TM, int TN>
+template <int EPI, int TM, int TN, int STAGES>
 __global__ __launch_bounds__(256) void linear_dma_kernel(pcb_linear_args a) {
     typedef bf16_t E;
     constexpr bool TWO = EPI == PCB_EPI_SILU_MUL;
     constexpr int BM = 32 * TM, BN = 32 * TN, ROWS = BM + (TWO ? 2 : 1) * BN, BK = 64;
     constexpr int NI = ROWS / 32;                                    // wave instructions per wave and stage
-    __shared__ __attribute__((aligned(16))) E img[2][ROWS * BK];
+    __shared__ __attribute__((aligned(16))) E img[STAGES][ROWS * BK];
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
     const int wm = wave >> 1, wn = wave & 1, group = lane >> 4, l15 = lane & 15;
     const int K = a.K, N = a.N;
@@ -440,12 +479,20 @@ __global__ __launch_bounds__(256) void linear_dma_kernel(pcb_linear_args a) {
         f.v = *reinterpret_cast<const u32x4*>(&img[buf][r * BK + ((4 * ks + group) ^ ((r >> 1) & 7)) * 8]);
         return f;
     };
-    fetch(0, 0);
+    // STAGES - 1 stages are in flight: at the top of a step the wave waits for its own part of the stage at hand (loads land in order),
+    // the barrier then says that everyone's has landed and that the buffer of the step before is read out
+#pragma unroll
+    for (int p = 0; p < STAGES - 1; ++p)
+        if (p * BK < K) fetch(p * BK, p);
     int buf = 0;
-    for (int k0 = 0; k0 < K; k0 += BK, buf ^= 1) {
-        asm volatile("s_waitcnt vmcnt(0)" ::: "memory");             // this wave's part of the stage has landed
-        __syncthreads();                                             // so has everyone's, and the other buffer is read out
-        if (k0 + BK < K) fetch(k0 + BK, buf ^ 1);
+    for (int k0 = 0; k0 < K; k0 += BK, buf = buf + 1 == STAGES ? 0 : buf + 1) {
+        if (STAGES > 2 && k0 + BK < K)
+            asm volatile("s_waitcnt vmcnt(%0) lgkmcnt(0)" ::"n"((STAGES - 2) * NI) : "memory");
+        else
+            asm volatile("s_waitcnt vmcnt(0) lgkmcnt(0)" ::: "memory");
+        __builtin_amdgcn_s_barrier();
+        asm volatile("" ::: "memory");
+        if (k0 + (STAGES - 1) * BK < K) fetch(k0 + (STAGES - 1) * BK, buf == 0 ? STAGES - 1 : buf - 1);
 #pragma unroll
         for (int ks = 0; ks < 2; ++ks) {
             Frag<E> fa[TM];
@@ -455,40 +502,124 @@ __global__ __launch_bounds__(256) void linear_dma_kernel(pcb_linear_args a) {
             for (int j = 0; j < TN; ++j) {
                 const Frag<E> fb = frag(buf, BM + (wn * TN + j) * 16 + l15, ks);
 #pragma unroll
-                for (int i = 0; i < TM; ++i) acc[i][j] = mma(fa[i], fb, acc[i][j]);
+                for (int i = 0; i < TM; ++i) acc[i][j] = mma(fb, fa[i], acc[i][j]);
                 if (TWO) {
                     const Frag<E> fb2 = frag(buf, BM + BN + (wn * TN + j) * 16 + l15, ks);
 #pragma unroll
-                    for (int i = 0; i < TM; ++i) acc2[i][j] = mma(fa[i], fb2, acc2[i][j]);
+                    for (int i = 0; i < TM; ++i) acc2[i][j] = mma(fb2, fa[i], acc2[i][j]);
                 }
             }
         }
     }
 
+    // (the weights are the products' first operand: a lane ends up with four neighbouring columns of one row.)
+    // Bias, gate and activation first, in the accumulators -- an activation is chosen once, around the loop over them --, then the stores
     const E* bias = (const E*)a.bias;
+    const E* bias2 = TWO ? (const E*)a.bias2 : nullptr;
 #pragma unroll
     for (int j = 0; j < TN; ++j) {
-        const int n = n_lo + (wn * TN + j) * 16 + l15;
-        if (n >= N) continue;
-        const float bv = bias ? to_f32(bias[n]) : 0.0f;
-        const float bv2 = (TWO && a.bias2) ? to_f32(((const E*)a.bias2)[n]) : 0.0f;
-        const float cs = (EPI == PCB_EPI_SCALE_ADD) ? a.col_scale[n] : 0.0f;
+        const int n = n_lo + (wn * TN + j) * 16 + 4 * group;
+        if (bias || TWO) {
+            float bv[4], bv2[4];
 #pragma unroll
-        for (int i = 0; i < TM; ++i)
-#pragma unroll
-            for (int r = 0; r < 4; ++r) {
-                const int m = m_lo + (wm * TM + i) * 16 + 4 * group + r;
-                if (m < m_hi) emit<E, EPI>(a, m, n, acc[i][j][r], TWO ? acc2[i][j][r] : 0.0f, bv, cs, bv2);
+            for (int e = 0; e < 4; ++e) {
+                const bool in = n + e < N;
+                bv[e] = bias && in ? to_f32(bias[n + e]) : 0.0f;
+                bv2[e] = TWO && bias2 && in ? to_f32(bias2[n + e]) : 0.0f;
             }
+#pragma unroll
+            for (int i = 0; i < TM; ++i) {
+                float rg = 1.0f;
+                if (TWO && a.row_gate) {
+                    const int m = m_lo + (wm * TM + i) * 16 + l15;
+                    rg = to_f32(((const E*)a.row_gate)[(m < m_hi ? m : m_hi - 1) * a.ld_row_gate]);
+                }
+#pragma unroll
+                for (int e = 0; e < 4; ++e) {
+                    acc[i][j][e] += bv[e];
+                    if (TWO) acc[i][j][e] = gate_act(a.act, acc[i][j][e]) * (acc2[TWO ? i : 0][TWO ? j : 0][e] + bv2[e]) * rg;
+                }
+            }
+        }
+    }
+    if (EPI == PCB_EPI_STORE && (a.act | a.act2)) {
+        const int end = act_end(a), mid = a.act_split > 0 && a.act_split < end ? a.act_split : end;
+        auto run = [&](auto code, int lo, int hi) {
+            constexpr int A = decltype(code)::value;
+#pragma unroll
+            for (int j = 0; j < TN; ++j) {
+                const int n = n_lo + (wn * TN + j) * 16 + 4 * group;
+#pragma unroll
+                for (int e = 0; e < 4; ++e)
+                    if (n + e >= lo && n + e < hi) {
+#pragma unroll
+                        for (int i = 0; i < TM; ++i) acc[i][j][e] = apply_act(A, acc[i][j][e], a.act_param);
+                    }
+            }
+        };
+        auto pass = [&](int act, int lo, int hi) {
+            if (n_lo >= hi || n_lo + BN <= lo) return;
+            switch (act) {
+                case PCB_ACT_SILU: run(std::integral_constant<int, PCB_ACT_SILU>{}, lo, hi); break;
+                case PCB_ACT_SIGMOID: run(std::integral_constant<int, PCB_ACT_SIGMOID>{}, lo, hi); break;
+                case PCB_ACT_RELU2: run(std::integral_constant<int, PCB_ACT_RELU2>{}, lo, hi); break;
+                case PCB_ACT_SOFTPLUS: run(std::integral_constant<int, PCB_ACT_SOFTPLUS>{}, lo, hi); break;
+                case PCB_ACT_SOFTCAP: run(std::integral_constant<int, PCB_ACT_SOFTCAP>{}, lo, hi); break;
+                case PCB_ACT_RELU: run(std::integral_constant<int, PCB_ACT_RELU>{}, lo, hi); break;
+                case PCB_ACT_GELU_TANH: run(std::integral_constant<int, PCB_ACT_GELU_TANH>{}, lo, hi); break;
+                case PCB_ACT_LOGSIGMOID: run(std::integral_constant<int, PCB_ACT_LOGSIGMOID>{}, lo, hi); break;
+                case PCB_ACT_SCALE: run(std::integral_constant<int, PCB_ACT_SCALE>{}, lo, hi); break;
+                default: break;
+            }
+        };
+#pragma unroll 1
+        for (int part = 0; part < 2; ++part) pass(part ? a.act2 : a.act, part ? mid : 0, part ? end : mid);
+    }
+    const int whole = act_end(a);                                    // columns that go to y
+    const int esz = (EPI == PCB_EPI_SCALE_ADD || a.out_f32) ? 4 : 2;
+    const bool quads = a.ldy % 4 == 0 && (uintptr_t)a.y % (4 * esz) == 0 && a.y_batch_stride % 4 == 0 &&
+                       (EPI != PCB_EPI_SCALE_ADD || !a.base || (a.ldbase % 4 == 0 && (uintptr_t)a.base % 16 == 0));
+    const int64_t y0 = a.n_batch > 0 ? (int64_t)blockIdx.z * a.y_batch_stride : 0;
+#pragma unroll
+    for (int j = 0; j < TN; ++j) {
+        const int n = n_lo + (wn * TN + j) * 16 + 4 * group;
+        float cs[4];
+#pragma unroll
+        for (int e = 0; e < 4; ++e) cs[e] = EPI == PCB_EPI_SCALE_ADD && n + e < N ? a.col_scale[n + e] : 0.0f;
+        const bool quad = quads && n + 4 <= whole;
+#pragma unroll
+        for (int i = 0; i < TM; ++i) {
+            const int m = m_lo + (wm * TM + i) * 16 + l15;
+            if (m >= m_hi) continue;
+            const f4 v = acc[i][j];
+            if (quad) {
+                if (EPI == PCB_EPI_SCALE_ADD) {
+                    f4* y = reinterpret_cast<f4*>((float*)a.y + (int64_t)m * a.ldy + n);
+                    const f4 b0 = a.base ? *reinterpret_cast<const f4*>(a.base + (int64_t)m * a.ldbase + n) : *y;
+                    *y = f4{b0[0] + cs[0] * v[0], b0[1] + cs[1] * v[1], b0[2] + cs[2] * v[2], b0[3] + cs[3] * v[3]};
+                } else {
+                    const int64_t at = (int64_t)(a.row_dst ? a.row_dst[m] : m) * a.ldy + n + y0;
+                    if (a.out_f32)
+                        *reinterpret_cast<f4*>((float*)a.y + at) = v;
+                    else
+                        *reinterpret_cast<uint2*>((E*)a.y + at) = uint2{(uint32_t)bf16_bits(v[0]) | ((uint32_t)bf16_bits(v[1]) << 16),
+                                                                        (uint32_t)bf16_bits(v[2]) | ((uint32_t)bf16_bits(v[3]) << 16)};
+                }
+            } else {
+#pragma unroll
+                for (int e = 0; e < 4; ++e)
+                    if (n + e < N) put<E, EPI>(a, m, n + e, v[e], cs[e]);
+            }
+        }
     }
 }
 
-template <int EPI, int TM, int TN>
+template <int EPI, int TM, int TN, int STAGES>
 int launch_dma(const pcb_linear_args& a, hipStream_t stream) {
     constexpr int BM = 32 * TM, BN = 32 * TN;
     const int nb = pcb_ceil_div(a.N, BN), mb = pcb_ceil_div(a.M, BM);
     const dim3 grid = a.n_groups > 0 ? dim3(nb, mb + a.n_groups) : dim3(8 * pcb_ceil_div(nb * mb, 8), 1, a.n_batch > 0 ? a.n_batch : 1);
-    hipLaunchKernelGGL((linear_dma_kernel<EPI, TM, TN>), grid, dim3(256), 0, stream, a);
+    hipLaunchKernelGGL((linear_dma_kernel<EPI, TM, TN, STAGES>), grid, dim3(256), 0, stream, a);
     return pcb_check_launch("linear_dma_kernel");
 }
 
@@ -505,10 +636,12 @@ int dispatch_dma(const pcb_linear_args& a, int rows, hipStream_t stream) {
     constexpr int TNW = EPI == PCB_EPI_SILU_MUL ? 2 : 4;
     const int64_t batch = a.n_batch > 0 ? a.n_batch : 1;
     auto tiles = [&](int bm, int bn) { return batch * pcb_ceil_div(a.M, bm) * pcb_ceil_div(a.N, bn); };
-    if (rows > 64 && tiles(128, 32 * TNW) >= 256) return launch_dma<EPI, 4, TNW>(a, stream);
-    if (rows > 32 && tiles(64, 32 * TNW) >= 256) return launch_dma<EPI, 2, TNW>(a, stream);
-    if (rows > 32) return launch_dma<EPI, 2, TNW / 2>(a, stream);
-    return launch_dma<EPI, 1, TNW / 2>(a, stream);
+    // (two workgroups of a CU hide each other's loads behind their products; a lone one needs a stage more in flight)
+    if (rows > 64 && tiles(128, 32 * TNW) > 256) return launch_dma<EPI, 4, TNW, 2>(a, stream);
+    if (rows > 64 && tiles(128, 32 * TNW) == 256) return launch_dma<EPI, 4, TNW, 3>(a, stream);
+    if (rows > 32 && tiles(64, 32 * TNW) >= 400) return launch_dma<EPI, 2, TNW, 3>(a, stream);
+    if (rows > 32) return launch_dma<EPI, 2, TNW / 2, 3>(a, stream);
+    return launch_dma<EPI, 1, TNW / 2, 3>(a, stream);
 }
 
 template <typename E, int EPI, int TM, int TN>
@@ -528,15 +661,18 @@ int dispatch(const pcb_linear_args& a, hipStream_t stream) {
     const bool big = rows > 64 && a.N > 64;
     if (rows <= 16) {
         const dim3 grid(pcb_ceil_div(a.N, 16), pcb_ceil_div(a.M, 16) + (a.n_groups > 0 ? a.n_groups : 0), a.n_batch > 0 ? a.n_batch : 1);
+        const bool deep = a.K >= 2048 && (int64_t)grid.x * grid.y * grid.z <= 192;
+        auto go = [&](auto epi) {
+            constexpr int EPI = decltype(epi)::value;
+            if (deep)
+                hipLaunchKernelGGL((linear_skinny_kernel<E, EPI, 16>), grid, dim3(64 * 16), 0, stream, a);
+            else
+                hipLaunchKernelGGL((linear_skinny_kernel<E, EPI, 8>), grid, dim3(64 * 8), 0, stream, a);
+        };
         switch (a.epilogue) {
-            case PCB_EPI_STORE:
-                hipLaunchKernelGGL((linear_skinny_kernel<E, PCB_EPI_STORE>), grid, dim3(64 * SKW), 0, stream, a);
-                break;
-            case PCB_EPI_SILU_MUL:
-                hipLaunchKernelGGL((linear_skinny_kernel<E, PCB_EPI_SILU_MUL>), grid, dim3(64 * SKW), 0, stream, a);
-                break;
-            default:
-                hipLaunchKernelGGL((linear_skinny_kernel<E, PCB_EPI_SCALE_ADD>), grid, dim3(64 * SKW), 0, stream, a);
+            case PCB_EPI_STORE: go(std::integral_constant<int, PCB_EPI_STORE>{}); break;
+            case PCB_EPI_SILU_MUL: go(std::integral_constant<int, PCB_EPI_SILU_MUL>{}); break;
+            default: go(std::integral_constant<int, PCB_EPI_SCALE_ADD>{});
         }
         return pcb_check_launch("linear_skinny_kernel");
     }
