@@ -228,6 +228,68 @@ def test_residual_step_takes_experts_and_leaves_the_stream_as_it_is(dtype, W_):
     assert torch.equal(both[:, W_:], x.to(dtype)) and bool((both[:, :W_] == 3.0).all()) and rel(x, f64(x0) + f64(y)) < 1e-7
 
 
+def matmul32(x, w):
+    return torch.matmul(x.float(), w.float().t().contiguous())
+
+
+@pytest.mark.parametrize("M,N", [(2048, 2048), (2000, 2300), (1000, 3300), (300, 1100), (130, 80), (40, 200), (29, 264)])
+@pytest.mark.parametrize("K", [8, 72, 200, 1032])
+def test_many_row_projections_at_every_tile_shape_and_their_edges(M, N, K):
+    """bf16 panels that travel to LDS by themselves: k ranges that end inside a stage (and before the ring is full), row and column counts
+    that end inside a tile, grids that select each tile size; bias, an activation split inside a tile, gated units, rows gathered and
+    scattered, the scaled accumulation."""
+    b, bf = B(), torch.bfloat16
+    x, w, w2 = (rnd(r, K, dtype=bf, seed=i, scale=K ** -0.25) for i, r in ((1, M), (2, N), (3, N)))
+    bias, bias2 = rnd(N, dtype=bf, seed=4), rnd(N, dtype=bf, seed=5)
+    z = matmul32(x, w) + bias.float()
+    y32, y16 = torch.zeros(M, N, device=DEV), torch.zeros(M, N + 4, dtype=bf, device=DEV)
+    b.linear(x, w, y32, M=M, bias=bias)
+    assert rel(y32, z) < 2e-6
+    cut = N // 2 + 3
+    b.linear(x, w, y16, M=M, bias=bias, act=b.ACT_SILU, act_split=cut, act2=b.ACT_SIGMOID, ldy=N + 4)
+    want = torch.cat([z[:, :cut] * torch.sigmoid(z[:, :cut]), torch.sigmoid(z[:, cut:])], dim=1)
+    assert rel(y16[:, :N], want) < 4e-3 and float(y16[:, N:].float().abs().max()) == 0.0
+    g = torch.zeros(M, N, dtype=bf, device=DEV)
+    for act, f in ((b.ACT_NONE, torch.nn.functional.silu), (b.ACT_RELU, torch.relu), (b.ACT_GELU_TANH, lambda t: torch.nn.functional.gelu(t, approximate="tanh"))):
+        b.linear(x, w, g, M=M, epilogue=b.EPI_SILU_MUL, w2=w2, bias=bias, bias2=bias2, act=act)
+        assert rel(g, f(z) * (matmul32(x, w2) + bias2.float())) < 4e-3
+    perm = torch.randperm(M, generator=torch.Generator().manual_seed(6)).to(torch.int32).to(DEV)
+    y32.zero_()
+    b.linear(x, w, y32, M=M, bias=bias, row_src=perm, row_dst=perm)
+    assert rel(y32, z) < 2e-6
+    base, cs = rnd(M, N, seed=7), rnd(N, seed=8)
+    b.linear(x, w, y32, M=M, bias=bias, epilogue=b.EPI_SCALE_ADD, base=base, col_scale=cs)
+    assert rel(y32, base + cs * z) < 2e-6
+
+
+@pytest.mark.parametrize("K", [64, 136])
+def test_many_row_projections_of_experts_and_split_destinations(K):
+    """Groups of unequal sizes (one empty, one of a single row) in a launch that takes the large tiles, and the three-way split store."""
+    b, bf, N = B(), torch.bfloat16, 264
+    sizes = [300, 0, 1, 130, 513]
+    M = sum(sizes)
+    x, w = rnd(M, K, dtype=bf, seed=1), rnd(len(sizes), N, K, dtype=bf, seed=2, scale=K ** -0.5)
+    off = dev_i32([0] + [sum(sizes[:i + 1]) for i in range(len(sizes))])
+    src = torch.randperm(M, generator=torch.Generator().manual_seed(3))
+    y = torch.zeros(M, N, device=DEV)
+    b.linear(x, w, y, M=M, row_src=src.to(torch.int32).to(DEV), group_off=off, n_groups=len(sizes))
+    want, at = [], 0
+    for g, n in enumerate(sizes):
+        want.append(matmul32(x[src.to(DEV)[at:at + n]], w[g]))
+        at += n
+    assert rel(y, torch.cat(want)) < 2e-6
+    # columns: 100 to rows, 84 to a cache of 3 heads kept row by row, 80 to one kept column by column
+    W1, R, cap = w[0], 500, 512
+    y1, y2 = torch.zeros(R, 100, dtype=bf, device=DEV), torch.zeros(3, cap, 28, dtype=bf, device=DEV)
+    y3 = torch.zeros(80, cap, dtype=bf, device=DEV)
+    pos = torch.randperm(cap, generator=torch.Generator().manual_seed(4))[:R].to(DEV)
+    b.linear(x, W1, y1, M=R, act=b.ACT_RELU2, split_n=100, y2=y2, row_off2=pos * 28, head_dim2=28, head_stride2=cap * 28, split_n3=184, y3=y3,
+             row_off3=pos.clone(), col_stride3=cap)
+    z = matmul32(x[:R], W1)
+    assert rel(y1, torch.relu(z[:, :100]) ** 2) < 5e-3
+    assert rel(y2[:, pos].permute(1, 0, 2).reshape(R, 84), z[:, 100:184]) < 5e-3 and rel(y3[:, pos].T, z[:, 184:]) < 5e-3
+
+
 def test_router_scores_are_not_renormalised():
     b, T, n, top = B(), 9, 11, 4
     z = rnd(T, n, seed=3, scale=2.0)
