@@ -23,7 +23,7 @@ import torch
 
 from ..pml import Preprocessor, PreprocessorList, escape_xml  # noqa: F401  (re-exported like the reference)
 from .config import (FALCON_SHAPES, MPT_SHAPES, SHAPES, BepepelShape, DibizenShape, FalconShape, FivesunShape, KazolornShape, LlamaShape, MptShape,
-                     PikadraShape, architecture_of)
+                     PikadraShape, VenitarShape, architecture_of)
 from .tokenizer import StandInTokenizer
 
 # HF hub ids the reference's drivers use (demo.py:27, eval.py:36, config/*.json) -> shape presets
@@ -481,8 +481,50 @@ class Pikadra(LanguageModel):
         return [t % self.config.vocab_size for t in super().encode(text)]
 
 
+class Venitar(LanguageModel):
+    """Adapter of the Venitar design (``config.VenitarShape``, ``venitar_hip.VenitarHIP``).  A checkpoint directory holds
+    ``config.json`` and ``model.safetensors``; without one, ``shape=`` plus ``random_init=True`` (or ``weights=``) gives seeded
+    random weights.  ``dtype``: ``torch.bfloat16`` (serving) or ``torch.float32`` (everything in true 32-bit)."""
+
+    def __init__(self, name: Optional[str] = None, device: str = "cuda:0", shape: Optional[VenitarShape] = None,
+                 weights=None, tokenizer=None, random_init: bool = False, seed: int = 0, dtype=torch.bfloat16, **_kwargs):
+        from .venitar_hip import VenitarHIP
+        from . import weights as W
+
+        if weights is not None:
+            assert shape is not None, "pass shape= together with weights="
+        elif name is not None and os.path.isdir(name):
+            shape = shape or VenitarShape.from_dir(name)
+            weights = W.load_venitar_safetensors(name, shape)
+        else:
+            if shape is None or not random_init:
+                raise FileNotFoundError(f"no checkpoint directory {name!r}: pass one, or shape= with random_init=True")
+            weights = W.make_venitar_weights(shape, seed, device=device)
+        if tokenizer is None:
+            tokenizer = StandInTokenizer(max(shape.vocab_size, 512))
+        model = VenitarHIP(shape, weights, device=device, dtype=dtype)
+        self.formatter = FormatConversation(system=("", "\n\n", ""), user=("User: ", "\n\nAssistant:"), assistant=(" ", "\n\n"))
+        super().__init__(name or shape.name, model, tokenizer, [tokenizer.eos_token_id], [])
+
+    def get_formatter(self) -> Callable[[str], str]:
+        return self.formatter
+
+    def get_cache_shape(self) -> Tuple[int, int, int]:
+        """(layer runs, kv heads, key size) of the first layer that keeps rows per token (zeros when none does); the recurrent mixers
+        keep states of their own shapes (``VenitarHIP.new_arena`` knows them all)."""
+        n = len(self.config.runs())
+        for l in self.config.layers:
+            if l.kind != "retention":
+                a = l.mix or l.left
+                return n, a.kv_heads, a.dim
+        return n, 0, 0
+
+    def encode(self, text: str) -> List[int]:
+        return [t % self.config.vocab_size for t in super().encode(text)]
+
+
 ADAPTERS = {"llama": Llama2, "falcon": Falcon, "mpt": Mpt, "kazolorn": Kazolorn, "dibizen": Dibizen, "fivesun": Fivesun,
-            "bepepel": Bepepel, "pikadra": Pikadra}
+            "bepepel": Bepepel, "pikadra": Pikadra, "venitar": Venitar}
 
 
 def load_language_model(path: str, **kwargs) -> LanguageModel:

@@ -7,7 +7,7 @@ from __future__ import annotations
 
 import json
 import os
-from dataclasses import dataclass, asdict
+from dataclasses import asdict, dataclass, field
 from typing import Optional
 
 
@@ -1020,6 +1020,257 @@ class PikadraShape:
         return s
 
 
+@dataclass
+class VenitarRot:
+    """Rotary positions of a Venitar mixer: the first ``dims`` columns of a head turn in halves (column i with column i + dims / 2),
+    base^(-2i / dims) radians per position; ``scaling``: None, or (factor, original, fast, slow) of the YaRN frequency ramp."""
+    base: float = 10000.0
+    dims: int = 0
+    scaling: Optional[tuple] = None
+
+    @classmethod
+    def from_config(cls, rot) -> "VenitarRot":
+        if not rot:
+            return cls()
+        sc = rot.get("scaling")
+        return cls(base=float(rot["base"]), dims=int(rot["dims"]),
+                   scaling=(float(sc["factor"]), float(sc["original"]), float(sc["fast"]), float(sc["slow"])) if sc else None)
+
+    def to_config(self) -> dict:
+        c = {"base": self.base, "dims": self.dims}
+        if self.scaling:
+            c["scaling"] = dict(zip(("factor", "original", "fast", "slow"), self.scaling))
+        return c
+
+
+@dataclass
+class VenitarRetention:
+    """Linear attention with one constant decay per head (``decay``, as long as there are heads), a ``dim`` x ``vdim`` matrix state
+    each, rotary queries and keys, per-head unit-RMS outputs behind a SiLU gate."""
+    heads: int
+    dim: int
+    vdim: int
+    decay: list
+    rot: VenitarRot = field(default_factory=VenitarRot)
+
+
+@dataclass
+class VenitarAttention:
+    """Softmax attention, ``heads`` query heads over ``kv_heads`` key heads.  As a layer's mixer: queries and keys normed per head with
+    gains, the values are the projected keys themselves, a key is seen inside the query's own block of ``block`` positions only (0: no
+    blocks), one more exp(0) in the denominator.  As the left half of a ``parallel`` mixer: biased projections, a sliding window of
+    ``window`` positions (0: none), an element-wise sigmoid gate."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    block: int = 0
+    window: int = 0
+    rot: VenitarRot = field(default_factory=VenitarRot)
+
+
+@dataclass
+class VenitarDelta:
+    """The right half of a ``parallel`` mixer: a gated delta rule, ``heads`` matrix states of ``dim`` x ``vdim`` whose queries and keys
+    come from ``kv_heads`` heads, a causal convolution of ``conv`` taps per channel on q, k and v, a decay per head and key channel
+    (low rank ``a_rank``) and a sigmoid output gate (low rank ``g_rank``).  The ranks are tensor shapes and are filled in by the weight
+    loader (0: not known yet)."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    conv: int
+    a_rank: int = 0
+    g_rank: int = 0
+
+    @property
+    def conv_channels(self) -> int:
+        return 2 * self.kv_heads * self.dim + self.heads * self.vdim
+
+
+@dataclass
+class VenitarLayer:
+    """One layer of a Venitar stack: ``kind`` "retention" (``mix``: ``VenitarRetention``), "attention" (``mix``: ``VenitarAttention``) or
+    "parallel" (``left``: ``VenitarAttention`` and ``right``: ``VenitarDelta`` on the same input, their results added with the weights
+    ``left_scale`` and ``right_scale``); ``ff`` > 0: a squared-ReLU feed-forward of that width behind it."""
+    kind: str
+    mix: object = None
+    left: Optional[VenitarAttention] = None
+    right: Optional[VenitarDelta] = None
+    left_scale: float = 1.0
+    right_scale: float = 1.0
+    ff: int = 0
+
+
+@dataclass
+class VenitarShape:
+    """Venitar: decoder-only, pre-norm layers (RMS norms) of three kinds of mixer, a run of layers that repeats ``loop_times`` times with
+    the same weights -- each pass with a cache and states of its own, every pass but the first entered by adding the embedding output
+    to the stream --, scaled embeddings whose table is the output projection as well.  Every size and constant comes from
+    ``config.json`` (``from_config``); ``loop_times`` 0: no layer repeats."""
+    vocab_size: int
+    hidden_size: int
+    norm_eps: float
+    layers: list
+    embed_scale: float = 1.0
+    loop_start: int = 0
+    loop_stop: int = 0
+    loop_times: int = 0
+    name: str = "venitar"
+
+    ARCHITECTURE = "Venitar"
+    KINDS = ("retention", "attention", "parallel")
+
+    @property
+    def num_hidden_layers(self) -> int:
+        return len(self.layers)
+
+    def runs(self) -> list:
+        """The layer runs of one forward in order: (layer, whether the embedding output joins the stream right before this run)."""
+        if not self.loop_times:
+            return [(i, False) for i in range(len(self.layers))]
+        out = [(i, False) for i in range(self.loop_start)]
+        for t in range(self.loop_times):
+            out += [(i, t > 0 and i == self.loop_start) for i in range(self.loop_start, self.loop_stop)]
+        return out + [(i, False) for i in range(self.loop_stop, len(self.layers))]
+
+    @classmethod
+    def from_config(cls, c: dict, name: str = "venitar") -> "VenitarShape":
+        if c.get("architecture") != cls.ARCHITECTURE:
+            raise ValueError(f"config.json describes {c.get('architecture')!r}, not {cls.ARCHITECTURE}")
+
+        def attention(a, mask_as):
+            heads, dim = int(a["heads"]), int(a["dim"])
+            return VenitarAttention(heads=heads, kv_heads=int(a.get("kv_heads") or heads), dim=dim, vdim=int(a.get("vdim") or dim),
+                                    scale=float(a["scale"]), rot=VenitarRot.from_config(a.get("rot")),
+                                    **{mask_as: int((a.get("mask") or {}).get("size") or 0)})
+
+        layers = []
+        for i, lc in enumerate(c["layers"]):
+            kind, m = lc.get("type"), lc.get("mixer") or {}
+            if kind == "retention":
+                dim = int(m["dim"])
+                lay = VenitarLayer(kind, mix=VenitarRetention(heads=int(m["heads"]), dim=dim, vdim=int(m.get("vdim") or dim),
+                                                              decay=[float(v) for v in m["decay"]], rot=VenitarRot.from_config(m.get("rot"))))
+            elif kind == "attention":
+                lay = VenitarLayer(kind, mix=attention(m, "block"))
+            elif kind == "parallel":
+                b = m["right"]
+                heads, dim = int(b["heads"]), int(b["dim"])
+                lay = VenitarLayer(kind, left=attention(m["left"], "window"), left_scale=float(m["left_scale"]),
+                                   right_scale=float(m["right_scale"]),
+                                   right=VenitarDelta(heads=heads, kv_heads=int(b.get("kv_heads") or heads), dim=dim,
+                                                      vdim=int(b.get("vdim") or dim), conv=int(b["conv"])))
+            else:
+                raise ValueError(f"layer {i}: unknown mixer type {kind!r}")
+            mlp = lc.get("mlp")
+            if mlp:
+                if mlp.get("kind", "dense") != "dense":
+                    raise ValueError(f"layer {i}: unknown feed-forward kind {mlp['kind']!r}")
+                lay.ff = int(mlp["ff"])
+                if lay.ff < 1:
+                    raise ValueError(f"layer {i}: a feed-forward of width {lay.ff}")
+            layers.append(lay)
+        loop = c.get("loop") or {}
+        shape = cls(vocab_size=int(c["vocab"]), hidden_size=int(c["width"]), norm_eps=float(c["norm"]["eps"]), layers=layers,
+                    embed_scale=float((c.get("embedding") or {}).get("scale", 1.0)), loop_start=int(loop.get("start", 0)),
+                    loop_stop=int(loop.get("stop", len(layers))) if loop else 0, loop_times=int(loop.get("times", 1)) if loop else 0, name=name)
+        shape.check()
+        return shape
+
+    def check(self) -> None:
+        def attention(i, a):
+            if min(a.heads, a.kv_heads, a.dim, a.vdim) < 1 or a.heads % a.kv_heads:
+                raise ValueError(f"layer {i}: {a.heads} query heads over {a.kv_heads} key heads of {a.dim} / {a.vdim} columns")
+            if min(a.block, a.window) < 0:
+                raise ValueError(f"layer {i}: a mask of negative size")
+            rotation(i, a)
+
+        def rotation(i, m):
+            if m.rot.dims % 2 or not 0 <= m.rot.dims <= m.dim:
+                raise ValueError(f"layer {i}: {m.rot.dims} rotated columns of {m.dim}")
+
+        for i, l in enumerate(self.layers):
+            if l.kind == "retention":
+                m = l.mix
+                if min(m.heads, m.dim, m.vdim) < 1 or len(m.decay) != m.heads or not all(0.0 <= d <= 1.0 for d in m.decay):
+                    raise ValueError(f"layer {i}: retention needs heads, sizes and a decay between 0 and 1 for each head")
+                rotation(i, m)
+            elif l.kind == "attention":
+                attention(i, l.mix)
+                if l.mix.vdim != l.mix.dim:
+                    raise ValueError(f"layer {i}: the values are the keys, so their sizes must agree ({l.mix.dim} / {l.mix.vdim})")
+            elif l.kind == "parallel":
+                attention(i, l.left)
+                b = l.right
+                if min(b.heads, b.kv_heads, b.dim, b.vdim, b.conv) < 1 or b.heads % b.kv_heads:
+                    raise ValueError(f"layer {i}: {b.heads} heads over {b.kv_heads} key heads, {b.conv} taps")
+            else:
+                raise ValueError(f"layer {i}: unknown mixer type {l.kind!r}")
+        if self.loop_times < 0 or (self.loop_times and not 0 <= self.loop_start < self.loop_stop <= len(self.layers)):
+            raise ValueError(f"layers {self.loop_start} .. {self.loop_stop} of {len(self.layers)} cannot run {self.loop_times} times")
+
+    @classmethod
+    def from_dir(cls, path: str) -> "VenitarShape":
+        with open(os.path.join(path, "config.json")) as f:
+            return cls.from_config(json.load(f), name=os.path.basename(os.path.normpath(path)))
+
+    def to_config(self) -> dict:
+        """The ``config.json`` form (what ``from_config`` reads)."""
+        def attention(a, size):
+            c = {"dim": a.dim, "heads": a.heads, "kv_heads": a.kv_heads, "scale": a.scale, "vdim": a.vdim}
+            if size:
+                c["mask"] = {"size": size}
+            if a.rot.dims:
+                c["rot"] = a.rot.to_config()
+            return c
+
+        out = []
+        for l in self.layers:
+            if l.kind == "retention":
+                m = l.mix
+                mixer = {"decay": list(m.decay), "dim": m.dim, "heads": m.heads, "vdim": m.vdim}
+                if m.rot.dims:
+                    mixer["rot"] = m.rot.to_config()
+            elif l.kind == "attention":
+                mixer = attention(l.mix, l.mix.block)
+            else:
+                b = l.right
+                mixer = {"left": attention(l.left, l.left.window), "left_scale": l.left_scale, "right_scale": l.right_scale,
+                         "right": {"conv": b.conv, "dim": b.dim, "heads": b.heads, "kv_heads": b.kv_heads, "vdim": b.vdim}}
+            out.append({"type": l.kind, "mixer": mixer, "mlp": {"ff": l.ff, "kind": "dense"} if l.ff else None})
+        c = {"architecture": self.ARCHITECTURE, "embedding": {"scale": self.embed_scale}, "layers": out, "norm": {"eps": self.norm_eps},
+             "vocab": self.vocab_size, "width": self.hidden_size}
+        if self.loop_times:
+            c["loop"] = {"start": self.loop_start, "stop": self.loop_stop, "times": self.loop_times}
+        return c
+
+    @classmethod
+    def uniform(cls, vocab: int, width: int, kinds, heads: int, kv_heads: int, dim: int, ff: int, block: int = 0, window: int = 0, conv: int = 4,
+                rank: int = 0, loop=None, name: str = "venitar") -> "VenitarShape":
+        """A stack whose mixers (``kinds``, one per layer) all have the same head sizes.  ``rank``: of the delta rule's low-rank
+        projections (0: a head's size).  ``loop``: (start, stop, times)."""
+        rot = VenitarRot(base=50000.0, dims=dim)
+        layers = []
+        for kind in kinds:
+            if kind == "retention":
+                lay = VenitarLayer(kind, mix=VenitarRetention(heads, dim, dim, [1.0 - 2.0 ** (-5.0 - 6.0 * h / max(heads - 1, 1)) for h in range(heads)],
+                                                              rot))
+            elif kind == "attention":
+                lay = VenitarLayer(kind, mix=VenitarAttention(heads, kv_heads, dim, dim, dim ** -0.5, block=block, rot=rot))
+            else:
+                lay = VenitarLayer(kind, left=VenitarAttention(heads, kv_heads, dim, dim, dim ** -0.5, window=window, rot=rot),
+                                   right=VenitarDelta(heads, heads, dim, dim, conv, rank or dim, rank or dim), left_scale=0.9, right_scale=1.2)
+            lay.ff = ff
+            layers.append(lay)
+        start, stop, times = loop or (0, 0, 0)
+        s = cls(vocab_size=vocab, hidden_size=width, norm_eps=1e-6, layers=layers, embed_scale=width ** 0.5, loop_start=start, loop_stop=stop,
+                loop_times=times, name=name)
+        s.check()
+        return s
+
+
 def architecture_of(path: str) -> str:
     """Which model family a checkpoint directory holds: ``architecture`` (Kazolorn) or HF's ``model_type``."""
     with open(os.path.join(path, "config.json")) as f:
@@ -1032,6 +1283,8 @@ def architecture_of(path: str) -> str:
         return "fivesun"
     if c.get("architecture") == BepepelShape.ARCHITECTURE:
         return "bepepel"
+    if c.get("architecture") == VenitarShape.ARCHITECTURE:
+        return "venitar"
     if c.get("architecture") == PikadraShape.ARCHITECTURE:
         return "pikadra"
     return str(c.get("model_type", "llama"))

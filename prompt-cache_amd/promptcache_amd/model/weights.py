@@ -699,3 +699,91 @@ def load_pikadra_safetensors(path: str, cfg):
         if tuple(raw[k].shape) != tuple(shp):
             raise ValueError(f"{path}: {k} has shape {tuple(raw[k].shape)}, the configuration implies {tuple(shp)}")
     return {k: raw[k] for k in want}
+
+
+def venitar_weight_shapes(cfg) -> Dict[str, tuple]:
+    """Tensor names and shapes of a Venitar checkpoint (``model.safetensors``): ``embed`` (also the output projection); per layer
+    ``l{i}.norm1`` and the mixer's ``l{i}.mix.*`` -- retention: ``q k v g o``; attention: ``q k q.norm k.norm o``; parallel:
+    ``left.q|k|v`` with ``.b``, ``left.g|o``, ``right.q|k|v`` with ``.conv``, ``right.b A_log norm a1 a2 dt_bias g1 g2 o`` --, with a
+    feed-forward ``l{i}.norm2`` and ``l{i}.mlp.up|down``; then ``final.norm``."""
+    W = cfg.hidden_size
+    s = {"embed": (cfg.vocab_size, W)}
+    for i, l in enumerate(cfg.layers):
+        p, m = f"l{i}.", f"l{i}.mix."
+        s[p + "norm1"] = (W,)
+        if l.kind == "retention":
+            HD, HV = l.mix.heads * l.mix.dim, l.mix.heads * l.mix.vdim
+            s[m + "q"], s[m + "k"], s[m + "v"], s[m + "g"], s[m + "o"] = (HD, W), (HD, W), (HV, W), (HV, W), (W, HV)
+        elif l.kind == "attention":
+            a = l.mix
+            s[m + "q"], s[m + "k"], s[m + "o"] = (a.heads * a.dim, W), (a.kv_heads * a.dim, W), (W, a.heads * a.vdim)
+            s[m + "q.norm"] = s[m + "k.norm"] = (a.dim,)
+        else:
+            a, b = l.left, l.right
+            for nm, n in (("q", a.heads * a.dim), ("k", a.kv_heads * a.dim), ("v", a.kv_heads * a.vdim)):
+                s[m + "left." + nm], s[m + "left." + nm + ".b"] = (n, W), (n,)
+            s[m + "left.g"], s[m + "left.o"] = (a.heads * a.vdim, W), (W, a.heads * a.vdim)
+            r, HD, HV = m + "right.", b.heads * b.dim, b.heads * b.vdim
+            for nm, n in (("q", b.kv_heads * b.dim), ("k", b.kv_heads * b.dim), ("v", HV)):
+                s[r + nm], s[r + nm + ".conv"] = (n, W), (n, b.conv)
+            s[r + "b"], s[r + "A_log"], s[r + "norm"], s[r + "o"] = (b.heads, W), (b.heads,), (b.vdim,), (W, HV)
+            s[r + "a1"], s[r + "a2"], s[r + "dt_bias"] = (b.a_rank, W), (HD, b.a_rank), (HD,)
+            s[r + "g1"], s[r + "g2"] = (b.g_rank, W), (HV, b.g_rank)
+        if l.ff:
+            s[p + "norm2"], s[p + "mlp.up"], s[p + "mlp.down"] = (W,), (l.ff, W), (W, l.ff)
+    s["final.norm"] = (W,)
+    return s
+
+
+def make_venitar_weights(cfg, seed: int = 0, device="cpu", scale: float = 1.0):
+    """Seeded random weights (bfloat16 torch tensors) with nothing at a value that would hide a dropped term: gains scattered around
+    one, non-zero biases, decay rates and step biases that let a head's channels forget over a few to hundreds of tokens."""
+    import torch
+    g = torch.Generator(device="cpu").manual_seed(seed)
+    on_gpu = str(device) != "cpu"
+    gd = torch.Generator(device=device).manual_seed(seed) if on_gpu else g
+
+    def rnd(shape, big=False):
+        if big and on_gpu:
+            return torch.randn(shape, generator=gd, device=device, dtype=torch.float32)
+        return torch.randn(shape, generator=g, dtype=torch.float32).to(device)
+
+    out = {}
+    for name, shp in venitar_weight_shapes(cfg).items():
+        leaf = name.rsplit(".", 1)[-1]
+        if leaf in ("norm", "norm1", "norm2"):
+            w = 1.0 + 0.2 * rnd(shp)
+        elif leaf == "conv":
+            w = rnd(shp) / (shp[-1] ** 0.5)
+        elif leaf == "A_log":
+            w = 0.7 * rnd(shp)
+        elif leaf == "dt_bias":
+            w = -3.0 + 1.2 * rnd(shp)
+        elif leaf == "b" and len(shp) == 1:
+            w = 0.3 * rnd(shp)
+        elif leaf == "embed":
+            w = rnd(shp, big=True) / (shp[-1] ** 0.5)
+        else:
+            w = (scale / (shp[-1] ** 0.5)) * rnd(shp, big=True)
+        out[name] = w.to(torch.bfloat16)
+    return out
+
+
+def load_venitar_safetensors(path: str, cfg):
+    """The tensors of ``<path>/model.safetensors`` by their own names, on the host, checked against the shapes the configuration
+    implies.  The low ranks of the delta rule's decay and gate projections are not in the configuration: they are read off ``a1`` and
+    ``g1`` and written into ``cfg``."""
+    raw = read_checkpoint_dir(path)
+    for i, l in enumerate(cfg.layers):
+        if l.kind == "parallel":
+            r = f"l{i}.mix.right."
+            l.right.a_rank = int(raw[r + "a1"].shape[0]) if r + "a1" in raw else l.right.a_rank
+            l.right.g_rank = int(raw[r + "g1"].shape[0]) if r + "g1" in raw else l.right.g_rank
+    want = venitar_weight_shapes(cfg)
+    missing = [k for k in want if k not in raw]
+    if missing:
+        raise KeyError(f"{path}: tensors missing for this configuration: {missing[:6]}{' ...' if len(missing) > 6 else ''}")
+    for k, shp in want.items():
+        if tuple(raw[k].shape) != tuple(shp):
+            raise ValueError(f"{path}: {k} has shape {tuple(raw[k].shape)}, the configuration implies {tuple(shp)}")
+    return {k: raw[k] for k in want}
