@@ -16,7 +16,7 @@
 extern "C" {
 #endif
 
-#define PCB_ABI_VERSION 5
+#define PCB_ABI_VERSION 6
 #define PCB_OK 0
 #define PCB_ERR_ARG (-2001)
 #define PCB_ERR_HIP_BASE (-3000)
@@ -341,6 +341,9 @@ int pcb_decay_attn(const pcb_decay_attn_args* a, void* stream);
 int pcb_causal_conv(const void* x, int64_t ldx, const void* w, const void* bias, int32_t dtype, int32_t silu, const int32_t* row_meta,
                     const void* state, int64_t slot_stride, void* out, int64_t ldo, int32_t n_rows, int32_t C, int32_t taps,
                     void* stream);
+/* pcb_conv_step: both at once for steps that bring every request exactly one token (reqs as in pcb_decay_attn). */
+int pcb_conv_step(const void* x, int64_t ldx, const void* w, const void* bias, int32_t dtype, int32_t silu, const int32_t* reqs,
+                  int32_t n_reqs, void* state, int64_t slot_stride, void* out, int64_t ldo, int32_t C, int32_t taps, void* stream);
 int pcb_conv_state_update(const void* x, int64_t ldx, int32_t dtype, const int32_t* reqs, int32_t n_reqs, void* state,
                           int64_t slot_stride, int32_t C, int32_t taps, void* stream);
 
@@ -396,6 +399,7 @@ int pcb_state_chain(const float* local, float* start, float* state, int64_t slot
  *   read (out given): out[r] = x[src] / sqrt(mean(x[src]^2) + eps) * gain as E;  x_out[r] = x[src] (fp32) if given
  *                     gain null: out[r] = x[src] as E, without a norm
  *                     layer_norm: out[r] = (x - mean(x)) / sqrt(mean((x - mean(x))^2) + eps) * gain + bias instead
+ * add (fp32 [..][width], optional, write half): x[src] also gains add[src], as it is (a stream's own beginning joins it again).
  * y_scale: the sublayer's result enters as y_scale * y (after gate and post norm; 1 = as it is).
  * src = rows ? rows[r] : r.  y fp32 [..][width]; gate E rows of stride ldg; x fp32 [..][width]; out rows ldo elements apart (0:
  * width).  width <= 16384. */
@@ -421,6 +425,7 @@ typedef struct pcb_post_norm_args {
     const float* pair_weight;
     int32_t pair_top;
     int64_t ldo;
+    const float* add;
 } pcb_post_norm_args;
 int pcb_post_norm(const pcb_post_norm_args* a, void* stream);
 
@@ -434,7 +439,8 @@ int pcb_post_norm(const pcb_post_norm_args* a, void* stream);
  *           (rot_half: the pair is columns rot_off + i, rot_off + rot_dims / 2 + i instead)
  *   store:  E at dst + (row_off ? row_off[row] : row * ld_dst) + h * head_stride + c * col_stride  (rows of a matrix, a cache kept
  *           row by row, or one kept column by column)
- * freqs: float64 [rot_dims / 2] on the device, shared by the segments that rotate (they have the same rot_dims).  head_dim <= 16384,
+ * freqs: float64 [rot_dims / 2] on the device, shared by the segments that rotate (they have the same rot_dims).  table (fp32
+ * [rows][rot_dims], optional): what pcb_rot_table left for these rows stands for pos, freqs and rot_mag.  head_dim <= 16384,
  * rot_dims <= 1024.  A segment may work in place (dst = src, the same strides). */
 typedef struct pcb_head_prep_seg {
     const void* src;
@@ -465,8 +471,13 @@ typedef struct pcb_head_prep_args {
     float eps;
     int32_t rot_half;
     pcb_head_prep_seg seg[4];
+    const float* table;
 } pcb_head_prep_args;
 int pcb_head_prep(const pcb_head_prep_args* a, void* stream);
+
+/* out[r] = mag * (cos a_0 .. cos a_(n-1) | sin a_0 .. sin a_(n-1)),  a_i = pos[r] * freqs[i] as a float64 product, n = n_pairs: the turns of
+ * a step's rows, once for all layers that rotate alike.  n_pairs <= 512. */
+int pcb_rot_table(const int32_t* pos, const double* freqs, float mag, float* out, int32_t n_rows, int32_t n_pairs, void* stream);
 
 /* Matrix memory with exponential gating (mLSTM): per (slot, head) a state S [dim][vdim], a normaliser n [dim] and a running
  * maximum m, all fp32, zero before position 0.  Per token, with the head's log input gate li and log forget gate lf:
@@ -558,8 +569,10 @@ int pcb_gla(const pcb_gla_args* a, void* stream);
  * (int32 x 4, device): key j of the request sits in row base + j of k and v, and the rows up to the tile's last query position
  * exist.  Query head h (column h * dim of its flat row) reads key head h / (H / Hkv).  The last tail_dim of the dim key columns may be
  * shared by all heads: they then come from row (tail_rows ? tail_rows[base + j] : base + j) of k_tail.  Key j is seen by the query
- * at position i iff j <= i and (window <= 0 or i - j < window).  sink (fp32 [H]) and gate (E, one number per row and head, stride
- * ldg): as in pcb_attn_softmax.  tile_rows: 64, or 128 (bf16).  dim <= 256, vdim <= 256. */
+ * at position i iff j <= i, (window <= 0 or i - j < window) and (block <= 0 or floor(i / block) == floor(j / block)).  sink (fp32 [H])
+ * and gate (E rows of stride ldg: one number per row and head, or one per element when gate_cols): as in pcb_attn_softmax.  slots: keys
+ * and values lie in a slot's cache instead -- t[0] is the slot, its keys start k_slot_stride, its values v_slot_stride elements after the
+ * slot before (no shared part then).  tile_rows: 64, or 128 (bf16).  dim <= 256, vdim <= 256. */
 typedef struct pcb_attn_prompt_args {
     uint32_t struct_bytes;
     int32_t dtype;
@@ -584,6 +597,10 @@ typedef struct pcb_attn_prompt_args {
     int64_t ldg;
     void* out;
     int64_t ldo;
+    int32_t block;
+    int32_t gate_cols;
+    int32_t slots;
+    int64_t k_slot_stride, v_slot_stride;
 } pcb_attn_prompt_args;
 int pcb_attn_prompt(const pcb_attn_prompt_args* a, void* stream);
 
@@ -613,6 +630,96 @@ typedef struct pcb_attn_latent_args {
     float* part;
 } pcb_attn_latent_args;
 int pcb_attn_latent(const pcb_attn_latent_args* a, void* stream);
+
+/* Causal softmax attention of single rows over a slot's cached keys and values (decoding; the query heads of one key head share a pass
+ * over its rows).  tile r = {slot, position, 1, flat row} (int32 x 4, device); key j of key head g of slot s: k + s * k_slot_stride +
+ * g * k_head_stride + j * k_row_stride, its value likewise behind v (keys and values may interleave in one plane).  Query head h reads key
+ * head h / (H / Hkv).  window, block, sink, gate (element-wise, or one number per row and head when gate_per_head) and n_splits (up to
+ * 64) as in pcb_attn_softmax; part: fp32 scratch of n_rows * H * n_splits * (vdim + 2) floats.  dim <= 256, vdim <= 256. */
+typedef struct pcb_attn_rows_args {
+    uint32_t struct_bytes;
+    int32_t dtype;
+    const void* q;
+    int64_t ldq;
+    const int32_t* tiles;
+    int32_t n_rows;
+    const void* k;
+    int64_t k_slot_stride, k_head_stride, k_row_stride;
+    const void* v;
+    int64_t v_slot_stride, v_head_stride, v_row_stride;
+    int32_t H, Hkv, dim, vdim;
+    float scale;
+    int32_t window;
+    int32_t block;
+    const float* sink;
+    const void* gate;
+    int64_t ldg;
+    int32_t gate_per_head;
+    void* out;
+    int64_t ldo;
+    int32_t n_splits;
+    float* part;
+} pcb_attn_rows_args;
+int pcb_attn_rows(const pcb_attn_rows_args* a, void* stream);
+
+/* Recurrences with a matrix state S [dim][vdim] per (slot, head), fp32, zero before position 0.  Per token and head h:
+ *   q = q_scale q^, k = k_scale k^        q^, k^: E rows with head h / (H / Hk) at column (h / (H / Hk)) * dim; unit_norm: divided by
+ *                                         sqrt(sum of squares + unit_eps); rot_dims > 0: turned in halves by the row's cosines and
+ *                                         sines (rot, fp32 [rows][rot_dims], see pcb_rot_table)
+ *   S <- diag(f) S                        f = decay[h] (a constant per head), or f_d = exp(ld_coef[h] * g(ld[row][h * dim + d])), a decay
+ *                                         per key channel and token from fp32 rows; g = ln(1 + e^z) when ld_softplus, else z; the
+ *                                         products must be <= 0 (ld_coef null: 1).  Exactly one of decay, ld is given.
+ *   u = beta given ? sigmoid(beta[row][h]) * (v - S^T k) : v      v: E rows, head h at column h * vdim; beta fp32 rows (the delta rule)
+ *   S <- S + k u^T;  o = S^T q
+ * Queries and keys stay fp32 from the norm and the turn on; decays, step sizes and all products are fp32.  request r = {slot, first
+ * position, tokens, first flat row} as in pcb_decay_attn; state fp32 [slots][H][dim][vdim] (slot_stride floats per slot).  dim <= 256.
+ *
+ * pcb_rec_prompt: any number of tokens, in chunks of 16: request r's chunks are consecutive records {first flat row, tokens (16, the
+ * last one fewer), 0, 0} of `chunks`, from index chunk0[r] on.  out fp32 [rows][ldo] = o.  scratch: pcb_rec_scratch(n_chunks, H, dim) floats.
+ * pcb_rec_step: every request brings one token; y (E rows of stride ldy) = o / sqrt(mean over the head of o^2 + eps) * gain (fp32 [vdim],
+ * null: 1) * gate (E rows of stride ldg, null: 1).  Heads that fit the registers of one workgroup only (pcb_rec_step_fits). */
+typedef struct pcb_rec_args {
+    uint32_t struct_bytes;
+    int32_t dtype;
+    const void* q;
+    const void* k;
+    const void* v;
+    int64_t ldq, ldk, ldv;
+    int32_t unit_norm;
+    float unit_eps;
+    const float* rot;
+    int32_t rot_dims;
+    float q_scale, k_scale;
+    const float* decay;
+    const float* ld;
+    int64_t ldld;
+    const float* ld_coef;
+    int32_t ld_softplus;
+    const float* beta;
+    int64_t ldbeta;
+    const int32_t* reqs;
+    int32_t n_reqs;
+    const int32_t* chunks;
+    const int32_t* chunk0;
+    int32_t n_chunks;
+    float* state;
+    int64_t slot_stride;
+    int32_t H, Hk, dim, vdim;
+    float* scratch;
+    int64_t scratch_floats;
+    float* out;
+    int64_t ldo;
+    const float* gain;
+    float eps;
+    const void* gate;
+    int64_t ldg;
+    void* y;
+    int64_t ldy;
+} pcb_rec_args;
+int64_t pcb_rec_scratch(int32_t n_chunks, int32_t H, int32_t dim);
+int pcb_rec_prompt(const pcb_rec_args* a, void* stream);
+int32_t pcb_rec_step_fits(int32_t dim, int32_t vdim);
+int pcb_rec_step(const pcb_rec_args* a, void* stream);
 
 #ifdef __cplusplus
 }

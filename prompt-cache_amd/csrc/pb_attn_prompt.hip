@@ -9,6 +9,7 @@
 // A wave's queries are its own from start to end, so nothing is merged at the end.  Waves whose queries all precede a block skip its
 // products; only blocks that straddle a query's own position or a window's edge pay for masks.  The keys' last tail_dim columns may be
 // shared by all heads (one rotated part per token): they are then fetched from rows of their own, through an index table if given.
+// Keys and values may also lie in a slot's cache, and a query may see its window or its block of positions only.
 // Workgroups of one head are neighbours eight apart in launch order: they share that head's keys and values in one XCD's L2.
 #include "pb_attn_common.h"
 
@@ -25,6 +26,13 @@ __device__ __forceinline__ u32x4 part_chunk(const E* p, int c, int c_lo, int c_h
 #pragma unroll
     for (int e = 0; e < CE; ++e) tmp[e] = (c + e >= c_lo && c + e < c_hi) ? p[c + e - c_lo] : from_f32<E>(0.0f);
     return *reinterpret_cast<u32x4*>(tmp);
+}
+
+// the oldest key the query at position i sees (it never moves back as i grows)
+__device__ __forceinline__ int oldest(const pcb_attn_prompt_args& a, int i) {
+    int lo = a.window > 0 && i - a.window + 1 > 0 ? i - a.window + 1 : 0;
+    if (a.block > 0) lo = max(lo, i / a.block * a.block);
+    return lo;
 }
 
 // KSQ: 32-element k-steps of the key size; VB: 16-column blocks of the value size; BK: keys per block
@@ -46,13 +54,14 @@ __global__ __launch_bounds__(64 * PW) void attn_prompt_kernel(pcb_attn_prompt_ar
     const int base = tile[0], pos0 = tile[1], rows = tile[2], row0 = tile[3];
     const int dim = a.dim, vdim = a.vdim, split = dim - a.tail_dim;  // columns [0, split) per head, [split, dim) shared
     const int last = pos0 + rows - 1;
-    const E* K = (const E*)a.k + (int64_t)base * a.k_row_stride + (int64_t)hk * a.k_head_stride;
-    const E* V = (const E*)a.v + (int64_t)base * a.v_row_stride + (int64_t)hk * a.v_head_stride;
+    const E* K = (const E*)a.k + (int64_t)base * (a.slots ? a.k_slot_stride : a.k_row_stride) + (int64_t)hk * a.k_head_stride;
+    const E* V = (const E*)a.v + (int64_t)base * (a.slots ? a.v_slot_stride : a.v_row_stride) + (int64_t)hk * a.v_head_stride;
     const E* KT = (const E*)a.k_tail;
     const int32_t* trow = a.tail_rows ? a.tail_rows + base : nullptr;
     // whether every 16-byte chunk of a row lies in one part and can be read at once
     const bool plain = ((uintptr_t)a.k % 16 == 0) && a.k_row_stride % CE == 0 && a.k_head_stride % CE == 0 && ((uintptr_t)a.v % 16 == 0) &&
                        a.v_row_stride % CE == 0 && a.v_head_stride % CE == 0 && dim % CE == 0 && vdim % CE == 0 && split % CE == 0 &&
+                       (!a.slots || (a.k_slot_stride % CE == 0 && a.v_slot_stride % CE == 0)) &&
                        (a.tail_dim == 0 || ((uintptr_t)a.k_tail % 16 == 0 && a.tail_row_stride % CE == 0));
 
     // this wave's queries
@@ -61,12 +70,13 @@ __global__ __launch_bounds__(64 * PW) void attn_prompt_kernel(pcb_attn_prompt_ar
     const int w_first = pos0 + w0, w_last = pos0 + (w0 + 16 * QT < rows ? w0 + 16 * QT : rows) - 1;
     const bool qvec = ((uintptr_t)a.q % 16 == 0) && (a.ldq % CE == 0) && (dim % CE == 0);
     Frag<E> qf[QT][KSQ];
-    int qpos[QT];
+    int qpos[QT], qlo[QT];
 #pragma unroll
     for (int qt = 0; qt < QT; ++qt) {
         int qi = w0 + 16 * qt + c;
         qi = qi < rows ? qi : rows - 1;                              // (lanes past the tile repeat its last query; nothing of theirs is stored)
         qpos[qt] = pos0 + qi;
+        qlo[qt] = oldest(a, pos0 + qi);
         const E* qp = (const E*)a.q + (int64_t)(row0 + qi) * a.ldq + (int64_t)h * dim;
 #pragma unroll
         for (int ks = 0; ks < KSQ; ++ks) qf[qt][ks] = load_frag(qp + 32 * ks, g, dim - 32 * ks, qvec);
@@ -83,7 +93,8 @@ __global__ __launch_bounds__(64 * PW) void attn_prompt_kernel(pcb_attn_prompt_ar
         for (int vb = 0; vb < VB; ++vb) o[qt][vb] = f4{0.f, 0.f, 0.f, 0.f};
     }
 
-    const int kb_lo = a.window > 0 && pos0 - a.window + 1 > 0 ? (pos0 - a.window + 1) / BK : 0;
+    const int kb_lo = oldest(a, pos0) / BK;
+    const int w_lo = oldest(a, w_first), w_lo_last = oldest(a, w_last);
     const int kb_hi = last / BK;
     u32x4 rk[KCH], rv[VCH];
     const int lr = tid / LPR, lc = tid % LPR * CE;                   // this thread's row and first column
@@ -133,7 +144,7 @@ __global__ __launch_bounds__(64 * PW) void attn_prompt_kernel(pcb_attn_prompt_ar
         __syncthreads();
         if (plain && kb < kb_hi) fetch(kb + 1);
         const int k0 = kb * BK;
-        if (!busy || k0 > w_last || (a.window > 0 && k0 + BK - 1 < w_first - a.window + 1)) continue;
+        if (!busy || k0 > w_last || k0 + BK - 1 < w_lo) continue;
 
         f4 s[QT][NKT];
 #pragma unroll
@@ -147,7 +158,7 @@ __global__ __launch_bounds__(64 * PW) void attn_prompt_kernel(pcb_attn_prompt_ar
                 for (int qt = 0; qt < QT; ++qt) s[qt][kt] = mma(kf, qf[qt][ks], s[qt][kt]);
             }
         }
-        const bool masked = k0 + BK - 1 > w_first || (a.window > 0 && k0 < w_last - a.window + 1);
+        const bool masked = k0 + BK - 1 > w_first || k0 < w_lo_last;
         PFrag<E> pf[QT][NK2];
 #pragma unroll
         for (int qt = 0; qt < QT; ++qt) {
@@ -159,7 +170,7 @@ __global__ __launch_bounds__(64 * PW) void attn_prompt_kernel(pcb_attn_prompt_ar
                     float v = s[qt][kt][r] * sc;
                     if (masked) {
                         const int key = k0 + kt * 16 + 4 * g + r;
-                        if (key > qpos[qt] || (a.window > 0 && qpos[qt] - key >= a.window)) v = NEG;
+                        if (key > qpos[qt] || key < qlo[qt]) v = NEG;
                     }
                     s[qt][kt][r] = v;
                     bm = fmaxf(bm, v);
@@ -215,18 +226,26 @@ __global__ __launch_bounds__(64 * PW) void attn_prompt_kernel(pcb_attn_prompt_ar
         }
         const int64_t qrow = row0 + w0 + 16 * qt + c;
         float f = keep / lt;
-        if (a.gate) f *= to_f32(((const E*)a.gate)[qrow * a.ldg + h]);
+        if (a.gate && !a.gate_cols) f *= to_f32(((const E*)a.gate)[qrow * a.ldg + h]);
+        const E* gp = a.gate && a.gate_cols ? (const E*)a.gate + qrow * a.ldg + (int64_t)h * vdim : nullptr;
         E* op = (E*)a.out + qrow * a.ldo + (int64_t)h * vdim;
         const bool ovec = ((uintptr_t)a.out % 16 == 0) && a.ldo % 4 == 0 && vdim % 4 == 0;
+        const bool gvec = gp && ((uintptr_t)a.gate % (4 * sizeof(E)) == 0) && a.ldg % 4 == 0 && vdim % 4 == 0;
 #pragma unroll
         for (int vb = 0; vb < VB; ++vb) {
             const int col = vb * 16 + 4 * g;
+            float gv[4] = {f, f, f, f};
+            if (gp) {
+                load4(gp + col, gvec, vdim - col, gv);
+#pragma unroll
+                for (int r = 0; r < 4; ++r) gv[r] *= f;
+            }
             if (ovec && col + 4 <= vdim) {
-                store4(op + col, o[qt][vb][0] * f, o[qt][vb][1] * f, o[qt][vb][2] * f, o[qt][vb][3] * f);
+                store4(op + col, o[qt][vb][0] * gv[0], o[qt][vb][1] * gv[1], o[qt][vb][2] * gv[2], o[qt][vb][3] * gv[3]);
             } else {
 #pragma unroll
                 for (int r = 0; r < 4; ++r)
-                    if (col + r < vdim) op[col + r] = from_f32<E>(o[qt][vb][r] * f);
+                    if (col + r < vdim) op[col + r] = from_f32<E>(o[qt][vb][r] * gv[r]);
             }
         }
     }
@@ -265,7 +284,9 @@ PCB_EXPORT int pcb_attn_prompt(const pcb_attn_prompt_args* a, void* stream) {
                 "pcb_attn_prompt: tiles of 64 rows, or 128 in bf16");
     if (a->n_tiles == 0) return PCB_OK;
     PCB_REQUIRE(a->q && a->tiles && a->k && a->v && a->out && (a->tail_dim == 0 || (a->k_tail && a->tail_row_stride >= a->tail_dim)) &&
-                    (!a->gate || a->ldg >= a->H),
+                    (!a->gate || a->ldg >= (a->gate_cols ? (int64_t)a->H * a->vdim : (int64_t)a->H)),
                 PCB_ERR_ARG, "pcb_attn_prompt: null pointer");
+    PCB_REQUIRE(!a->slots || (a->tail_dim == 0 && a->k_slot_stride >= 0 && a->v_slot_stride >= 0), PCB_ERR_ARG,
+                "pcb_attn_prompt: keys in slots have no shared part");
     return a->dtype == PCB_BF16 ? dispatch<pcb::bf16_t>(*a, (hipStream_t)stream) : dispatch<float>(*a, (hipStream_t)stream);
 }

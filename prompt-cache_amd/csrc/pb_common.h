@@ -144,6 +144,27 @@ __device__ __forceinline__ f4 mma(const Frag<float>& a, const Frag<float>& b, f4
     for (int e = 0; e < 8; ++e) c = __builtin_amdgcn_mfma_f32_16x16x4f32(a.v[e], b.v[e], c, 0, 0, 0);
     return c;
 }
+// four consecutive elements of a row as floats; `valid` of them exist (<= 0: none); `vec`: one 8- or 16-byte load is allowed
+__device__ __forceinline__ void load4(const bf16_t* p, bool vec, int valid, float (&o)[4]) {
+    if (vec && valid >= 4) {
+        const uint2 w = *reinterpret_cast<const uint2*>(p);
+        o[0] = __uint_as_float(w.x << 16), o[1] = __uint_as_float(w.x & 0xffff0000u);
+        o[2] = __uint_as_float(w.y << 16), o[3] = __uint_as_float(w.y & 0xffff0000u);
+    } else {
+#pragma unroll
+        for (int i = 0; i < 4; ++i) o[i] = i < valid ? to_f32(p[i]) : 0.0f;
+    }
+}
+__device__ __forceinline__ void load4(const float* p, bool vec, int valid, float (&o)[4]) {
+    if (vec && valid >= 4) {
+        const float4 w = *reinterpret_cast<const float4*>(p);
+        o[0] = w.x, o[1] = w.y, o[2] = w.z, o[3] = w.w;
+    } else {
+#pragma unroll
+        for (int i = 0; i < 4; ++i) o[i] = i < valid ? p[i] : 0.0f;
+    }
+}
+
 // result tile: lane l holds column (l & 15), rows 4 * (l >> 4) + r, r = 0..3
 
 }  // namespace pcb

@@ -97,7 +97,13 @@ __global__ __launch_bounds__(256) void head_prep_kernel(pcb_head_prep_args a) {
     const pcb_head_prep_seg& s = a.seg[blockIdx.y];
     const int64_t row = blockIdx.x;
     const int np = s.rot_dims / 2;
-    if (np > 0) {
+    if (np > 0 && a.table) {
+        for (int i = threadIdx.x; i < np; i += 256) {
+            cs[i] = a.table[row * s.rot_dims + i];
+            sn[i] = a.table[row * s.rot_dims + np + i];
+        }
+        __syncthreads();
+    } else if (np > 0) {
         const double p = (double)a.pos[row];
         for (int i = threadIdx.x; i < np; i += 256) {
             double sv, cv;
@@ -113,7 +119,28 @@ __global__ __launch_bounds__(256) void head_prep_kernel(pcb_head_prep_args a) {
         prep_heads<E, false>(a, s, row, cs, sn, red);
 }
 
+__global__ __launch_bounds__(256) void rot_table_kernel(const int32_t* __restrict__ pos, const double* __restrict__ freqs, float mag,
+                                                        float* __restrict__ out, int n_rows, int np) {
+    const int64_t e = (int64_t)blockIdx.x * 256 + threadIdx.x;
+    if (e >= (int64_t)n_rows * np) return;
+    const int64_t r = e / np;
+    const int i = (int)(e % np);
+    double sv, cv;
+    sincos((double)pos[r] * freqs[i], &sv, &cv);
+    out[r * 2 * np + i] = (float)cv * mag;
+    out[r * 2 * np + np + i] = (float)sv * mag;
+}
+
 }  // namespace
+
+PCB_EXPORT int pcb_rot_table(const int32_t* pos, const double* freqs, float mag, float* out, int32_t n_rows, int32_t n_pairs, void* stream) {
+    PCB_REQUIRE(n_rows >= 0 && n_pairs > 0 && n_pairs <= MAX_PAIRS, PCB_ERR_ARG, "pcb_rot_table: bad sizes (up to 512 pairs)");
+    if (n_rows == 0) return PCB_OK;
+    PCB_REQUIRE(pos && freqs && out, PCB_ERR_ARG, "pcb_rot_table: null pointer");
+    const int64_t blocks = ((int64_t)n_rows * n_pairs + 255) / 256;
+    hipLaunchKernelGGL(rot_table_kernel, dim3((uint32_t)blocks), dim3(256), 0, (hipStream_t)stream, pos, freqs, mag, out, n_rows, n_pairs);
+    return pcb_check_launch("rot_table_kernel");
+}
 
 PCB_EXPORT int pcb_head_prep(const pcb_head_prep_args* a, void* stream) {
     PCB_REQUIRE(a && a->struct_bytes == sizeof(pcb_head_prep_args), PCB_ERR_ARG, "pcb_head_prep: struct size mismatch");
@@ -133,7 +160,7 @@ PCB_EXPORT int pcb_head_prep(const pcb_head_prep_args* a, void* stream) {
         PCB_REQUIRE(a->n_rows == 0 || (s.src && s.dst), PCB_ERR_ARG, "pcb_head_prep: null pointer");
     }
     if (a->n_rows == 0) return PCB_OK;
-    PCB_REQUIRE(rot == 0 || (a->pos && a->freqs), PCB_ERR_ARG, "pcb_head_prep: a rotation needs positions and frequencies");
+    PCB_REQUIRE(rot == 0 || a->table || (a->pos && a->freqs), PCB_ERR_ARG, "pcb_head_prep: a rotation needs positions and frequencies");
     const dim3 grid(a->n_rows, a->n_segs);
     if (a->dtype == PCB_BF16)
         hipLaunchKernelGGL(head_prep_kernel<pcb::bf16_t>, grid, dim3(256), 0, (hipStream_t)stream, *a);

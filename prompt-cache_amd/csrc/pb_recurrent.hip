@@ -1,6 +1,8 @@
 // Mixers that carry a state from token to token instead of a key cache: linear attention with a scalar decay per head
 // (pcb_decay_attn), the short causal convolution (pcb_causal_conv, pcb_conv_state_update) and the selective scan
 // (pcb_selective_scan).  States, decays, step sizes and every product that feeds a state are fp32.
+#include <type_traits>
+
 #include "pb_common.h"
 
 namespace {
@@ -21,27 +23,6 @@ __device__ __forceinline__ float decay_pow(float log2_decay, int n) { return n <
 // all on the fp32 matrix cores (v_mfma_f32_16x16x4_f32), elements of E widened exactly.  The state tiles ARE the operand
 // fragments of S^T Q^T: the k index of that product runs over the key columns in the order (l >> 4, 4 i + u) -> 16 i + 4 (l >> 4) + u,
 // which the query operand follows.
-// four consecutive elements of a row as floats; `valid` of them exist (<= 0: none); `vec`: one 8- or 16-byte load is allowed
-__device__ __forceinline__ void load4(const bf16_t* p, bool vec, int valid, float (&o)[4]) {
-    if (vec && valid >= 4) {
-        const uint2 w = *reinterpret_cast<const uint2*>(p);
-        o[0] = __uint_as_float(w.x << 16), o[1] = __uint_as_float(w.x & 0xffff0000u);
-        o[2] = __uint_as_float(w.y << 16), o[3] = __uint_as_float(w.y & 0xffff0000u);
-    } else {
-#pragma unroll
-        for (int i = 0; i < 4; ++i) o[i] = i < valid ? to_f32(p[i]) : 0.0f;
-    }
-}
-__device__ __forceinline__ void load4(const float* p, bool vec, int valid, float (&o)[4]) {
-    if (vec && valid >= 4) {
-        const float4 w = *reinterpret_cast<const float4*>(p);
-        o[0] = w.x, o[1] = w.y, o[2] = w.z, o[3] = w.w;
-    } else {
-#pragma unroll
-        for (int i = 0; i < 4; ++i) o[i] = i < valid ? p[i] : 0.0f;
-    }
-}
-
 template <typename E, int NB>
 __global__ __launch_bounds__(64) void decay_attn_kernel(pcb_decay_attn_args a) {
     const int lane = threadIdx.x, g = lane >> 4, c = lane & 15;
@@ -195,6 +176,123 @@ __global__ __launch_bounds__(256) void causal_conv_kernel(const E* __restrict__ 
     }
     if (silu) acc = acc / (1.0f + expf(-acc));
     out[r * ldo + ch] = from_f32<E>(acc);
+}
+
+// the same for few taps: a thread owns two neighbouring channels and walks a run of rows, so that an input is read once
+constexpr int CONV_RUN = 8;
+__device__ __forceinline__ void load2(const bf16_t* p, float (&o)[2]) {
+    const uint32_t w = *reinterpret_cast<const uint32_t*>(p);
+    o[0] = __uint_as_float(w << 16), o[1] = __uint_as_float(w & 0xffff0000u);
+}
+__device__ __forceinline__ void load2(const float* p, float (&o)[2]) {
+    const float2 w = *reinterpret_cast<const float2*>(p);
+    o[0] = w.x, o[1] = w.y;
+}
+__device__ __forceinline__ void store2(bf16_t* p, float a, float b) {
+    *reinterpret_cast<uint32_t*>(p) = (uint32_t)bf16_bits(a) | ((uint32_t)bf16_bits(b) << 16);
+}
+__device__ __forceinline__ void store2(float* p, float a, float b) { *reinterpret_cast<float2*>(p) = float2{a, b}; }
+
+template <typename E, int TAPS>
+__global__ __launch_bounds__(256) void causal_conv_run_kernel(const E* __restrict__ x, int64_t ldx, const E* __restrict__ w,
+                                                              const E* __restrict__ bias, int silu, const int32_t* __restrict__ meta,
+                                                              const E* __restrict__ state, int64_t slot_stride, E* __restrict__ out,
+                                                              int64_t ldo, int n_rows, int C) {
+    const int r0 = blockIdx.x * CONV_RUN;
+    const int ch = (blockIdx.y * 256 + threadIdx.x) * 2;
+    if (ch >= C) return;
+    float wt[TAPS][2], b0[2] = {0.0f, 0.0f}, old[TAPS - 1][2];      // old[m]: the input m + 1 tokens back
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j) wt[j][0] = to_f32(w[(int64_t)ch * TAPS + j]), wt[j][1] = to_f32(w[(int64_t)(ch + 1) * TAPS + j]);
+    if (bias) b0[0] = to_f32(bias[ch]), b0[1] = to_f32(bias[ch + 1]);
+    float in[CONV_RUN][2];
+#pragma unroll
+    for (int i = 0; i < CONV_RUN; ++i) {
+        in[i][0] = in[i][1] = 0.0f;
+        if (r0 + i < n_rows) load2(x + (int64_t)(r0 + i) * ldx + ch, in[i]);
+    }
+#pragma unroll
+    for (int i = 0; i < CONV_RUN; ++i) {
+        const int64_t r = r0 + i;
+        if (r >= n_rows) break;
+        const int slot = meta[4 * r], pos = meta[4 * r + 1], idx = meta[4 * r + 2];
+        if (i == 0 || idx == 0) {                           // what lies before the run, or before the request's rows of this step
+#pragma unroll
+            for (int m = 0; m < TAPS - 1; ++m) {
+                const int back = m + 1;
+                old[m][0] = old[m][1] = 0.0f;
+                if (back <= idx)
+                    load2(x + (r - back) * ldx + ch, old[m]);
+                else if (pos - back >= 0)
+                    load2(state + (int64_t)slot * slot_stride + (int64_t)(TAPS - 1 - (back - idx)) * C + ch, old[m]);
+            }
+        }
+        float acc[2] = {b0[0], b0[1]};
+#pragma unroll
+        for (int j = 0; j < TAPS; ++j)
+#pragma unroll
+            for (int e = 0; e < 2; ++e) acc[e] += wt[j][e] * (j == TAPS - 1 ? in[i][e] : old[j == TAPS - 1 ? 0 : TAPS - 2 - j][e]);
+        if (silu)
+#pragma unroll
+            for (int e = 0; e < 2; ++e) acc[e] = acc[e] / (1.0f + expf(-acc[e]));
+        store2(out + r * ldo + ch, acc[0], acc[1]);
+#pragma unroll
+        for (int m = TAPS - 2; m > 0; --m) old[m][0] = old[m - 1][0], old[m][1] = old[m - 1][1];
+        old[0][0] = in[i][0], old[0][1] = in[i][1];
+    }
+}
+
+// one token per request: the convolution and the state's move in one pass (a thread owns its channel)
+template <typename E>
+__global__ __launch_bounds__(256) void conv_step_kernel(const E* __restrict__ x, int64_t ldx, const E* __restrict__ w, const E* __restrict__ bias,
+                                                        int silu, const int32_t* __restrict__ reqs, E* __restrict__ state, int64_t slot_stride,
+                                                        E* __restrict__ out, int64_t ldo, int C, int taps) {
+    const int32_t* rq = reqs + 4 * blockIdx.x;
+    const int slot = rq[0], pos = rq[1];
+    const int64_t r = rq[3];
+    const int ch = blockIdx.y * 256 + threadIdx.x;
+    if (ch >= C) return;
+    E* st = state + (int64_t)slot * slot_stride + ch;
+    const E* wc = w + (int64_t)ch * taps;
+    const int m1 = taps - 1;
+    const E xv = x[r * ldx + ch];
+    E old[MAX_TAPS];
+#pragma unroll
+    for (int m = 0; m < MAX_TAPS; ++m) {
+        if (m >= m1) break;
+        old[m] = pos - m1 + m >= 0 ? st[(int64_t)m * C] : from_f32<E>(0.0f);      // (state row m: the token m1 - m before this one)
+    }
+    float acc = bias ? to_f32(bias[ch]) : 0.0f;
+#pragma unroll
+    for (int m = 0; m < MAX_TAPS; ++m) {
+        if (m >= m1) break;
+        acc += to_f32(wc[m]) * to_f32(old[m]);
+        if (m > 0) st[(int64_t)(m - 1) * C] = old[m];
+    }
+    acc += to_f32(wc[m1]) * to_f32(xv);
+    if (m1 > 0) st[(int64_t)(m1 - 1) * C] = xv;
+    if (silu) acc = acc / (1.0f + expf(-acc));
+    out[r * ldo + ch] = from_f32<E>(acc);
+}
+
+// (two channels at a time: rows and channels that start at multiples of two elements)
+template <typename E>
+bool launch_conv_run(const void* x, int64_t ldx, const void* w, const void* bias, int silu, const int32_t* meta, const void* state, int64_t slot_stride,
+                     void* out, int64_t ldo, int n_rows, int C, int taps, hipStream_t stream) {
+    constexpr uintptr_t A2 = 2 * sizeof(E);
+    if (C % 2 || ldx % 2 || ldo % 2 || slot_stride % 2 || (uintptr_t)x % A2 || (uintptr_t)out % A2 || (uintptr_t)state % A2) return false;
+    const dim3 grid(pcb_ceil_div(n_rows, CONV_RUN), pcb_ceil_div(C, 512)), block(256);
+    auto go = [&](auto t) {
+        hipLaunchKernelGGL((causal_conv_run_kernel<E, decltype(t)::value>), grid, block, 0, stream, (const E*)x, ldx, (const E*)w, (const E*)bias, silu,
+                           meta, (const E*)state, slot_stride, (E*)out, ldo, n_rows, C);
+        return true;
+    };
+    switch (taps) {
+        case 2: return go(std::integral_constant<int, 2>{});
+        case 3: return go(std::integral_constant<int, 3>{});
+        case 4: return go(std::integral_constant<int, 4>{});
+        default: return false;
+    }
 }
 
 template <typename E>
@@ -392,6 +490,9 @@ PCB_EXPORT int pcb_causal_conv(const void* x, int64_t ldx, const void* w, const 
                 PCB_ERR_ARG, "pcb_causal_conv: bad sizes (1 <= taps <= 16)");
     if (n_rows == 0) return PCB_OK;
     PCB_REQUIRE(x && w && row_meta && out && (taps == 1 || state), PCB_ERR_ARG, "pcb_causal_conv: null pointer");
+    if (dtype == PCB_BF16 ? launch_conv_run<pcb::bf16_t>(x, ldx, w, bias, silu, row_meta, state, slot_stride, out, ldo, n_rows, C, taps, (hipStream_t)stream)
+                          : launch_conv_run<float>(x, ldx, w, bias, silu, row_meta, state, slot_stride, out, ldo, n_rows, C, taps, (hipStream_t)stream))
+        return pcb_check_launch("causal_conv_run_kernel");
     const dim3 grid(n_rows, pcb_ceil_div(C, 256));
     if (dtype == PCB_BF16)
         hipLaunchKernelGGL(causal_conv_kernel<pcb::bf16_t>, grid, dim3(256), 0, (hipStream_t)stream, (const pcb::bf16_t*)x, ldx,
@@ -401,6 +502,23 @@ PCB_EXPORT int pcb_causal_conv(const void* x, int64_t ldx, const void* w, const 
         hipLaunchKernelGGL(causal_conv_kernel<float>, grid, dim3(256), 0, (hipStream_t)stream, (const float*)x, ldx, (const float*)w,
                            (const float*)bias, silu, row_meta, (const float*)state, slot_stride, (float*)out, ldo, C, taps);
     return pcb_check_launch("causal_conv_kernel");
+}
+
+PCB_EXPORT int pcb_conv_step(const void* x, int64_t ldx, const void* w, const void* bias, int32_t dtype, int32_t silu, const int32_t* reqs,
+                             int32_t n_reqs, void* state, int64_t slot_stride, void* out, int64_t ldo, int32_t C, int32_t taps, void* stream) {
+    PCB_REQUIRE((dtype == PCB_BF16 || dtype == PCB_F32) && n_reqs >= 0 && C > 0 && taps >= 1 && taps <= MAX_TAPS && ldx >= C && ldo >= C &&
+                    slot_stride >= (int64_t)(taps - 1) * C,
+                PCB_ERR_ARG, "pcb_conv_step: bad sizes (1 <= taps <= 16)");
+    if (n_reqs == 0) return PCB_OK;
+    PCB_REQUIRE(x && w && reqs && out && (taps == 1 || state), PCB_ERR_ARG, "pcb_conv_step: null pointer");
+    const dim3 grid(n_reqs, pcb_ceil_div(C, 256));
+    if (dtype == PCB_BF16)
+        hipLaunchKernelGGL(conv_step_kernel<pcb::bf16_t>, grid, dim3(256), 0, (hipStream_t)stream, (const pcb::bf16_t*)x, ldx, (const pcb::bf16_t*)w,
+                           (const pcb::bf16_t*)bias, silu, reqs, (pcb::bf16_t*)state, slot_stride, (pcb::bf16_t*)out, ldo, C, taps);
+    else
+        hipLaunchKernelGGL(conv_step_kernel<float>, grid, dim3(256), 0, (hipStream_t)stream, (const float*)x, ldx, (const float*)w, (const float*)bias,
+                           silu, reqs, (float*)state, slot_stride, (float*)out, ldo, C, taps);
+    return pcb_check_launch("conv_step_kernel");
 }
 
 PCB_EXPORT int pcb_conv_state_update(const void* x, int64_t ldx, int32_t dtype, const int32_t* reqs, int32_t n_reqs, void* state,

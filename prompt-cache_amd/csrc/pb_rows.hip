@@ -438,7 +438,8 @@ __global__ __launch_bounds__(1024) void post_norm_kernel(pcb_post_norm_args a) {
     const int64_t src = a.rows ? a.rows[r] : r;
     float* __restrict__ x = a.x + src * W;
     float ss[1] = {0.0f};
-    if (a.y || a.pair) {
+    const float* __restrict__ add = a.add ? a.add + src * W : nullptr;
+    if (a.y || a.pair || add) {
         const float* __restrict__ y = a.y ? a.y + src * W : nullptr;
         const E* __restrict__ g = a.gate ? (const E*)a.gate + src * a.ldg : nullptr;
         const float* __restrict__ pair = a.pair ? a.pair + src * a.pair_top * W : nullptr;
@@ -459,7 +460,8 @@ __global__ __launch_bounds__(1024) void post_norm_kernel(pcb_post_norm_args a) {
         ss[0] = 0.0f;
         const float ys = a.y_scale;
         for (int c = threadIdx.x; c < W; c += blockDim.x) {          // (a thread meets its own columns again: no barrier needed)
-            const float v = x[c] + ys * (a.post_gain ? row[c] * inv * a.post_gain[c] : row[c]);
+            float v = x[c] + ys * (a.post_gain ? row[c] * inv * a.post_gain[c] : row[c]);
+            if (add) v += add[c];
             row[c] = v;
             if (!a.rows) x[c] = v;
             ss[0] += v * v;

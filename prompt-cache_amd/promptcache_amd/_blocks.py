@@ -19,7 +19,7 @@ EPI_STORE, EPI_SILU_MUL, EPI_SCALE_ADD = 0, 1, 2
 ACT_NONE, ACT_SILU, ACT_SIGMOID, ACT_RELU2, ACT_SOFTPLUS, ACT_SOFTCAP, ACT_RELU, ACT_GELU_TANH, ACT_LOGSIGMOID, ACT_SCALE = range(10)
 NORM_NONE, NORM_RMS, NORM_DYT = 0, 1, 2
 SCORE_SIGMOID, SCORE_SOFTMAX = 0, 1
-ABI_VERSION = 5
+ABI_VERSION = 6
 DTYPES = {torch.bfloat16: BF16, torch.float32: F32}
 
 
@@ -100,7 +100,7 @@ class PostNormArgs(C.Structure):
                 ("x", _vp), ("y", _vp), ("gate", _vp), ("ldg", _i64), ("post_gain", _vp), ("gain", _vp),
                 ("out", _vp), ("x_out", _vp), ("rows", _vp), ("eps", _f32), ("n_rows", _i32), ("width", _i32),
                 ("y_scale", _f32), ("layer_norm", _i32), ("bias", _vp),
-                ("pair", _vp), ("pair_weight", _vp), ("pair_top", _i32), ("ldo", _i64)]
+                ("pair", _vp), ("pair_weight", _vp), ("pair_top", _i32), ("ldo", _i64), ("add", _vp)]
 
 
 class HeadPrepSeg(C.Structure):
@@ -114,7 +114,8 @@ class HeadPrepSeg(C.Structure):
 class HeadPrepArgs(C.Structure):
     """``pcb_head_prep_args`` (field for field)."""
     _fields_ = [("struct_bytes", C.c_uint32), ("dtype", _i32), ("n_rows", _i32), ("n_segs", _i32),
-                ("pos", _vp), ("freqs", _vp), ("rot_mag", _f32), ("eps", _f32), ("rot_half", _i32), ("seg", HeadPrepSeg * 4)]
+                ("pos", _vp), ("freqs", _vp), ("rot_mag", _f32), ("eps", _f32), ("rot_half", _i32), ("seg", HeadPrepSeg * 4),
+                ("table", _vp)]
 
 
 class MlstmArgs(C.Structure):
@@ -144,7 +145,8 @@ class AttnPromptArgs(C.Structure):
                 ("k_tail", _vp), ("tail_row_stride", _i64), ("tail_rows", _vp), ("tail_dim", _i32),
                 ("v", _vp), ("v_row_stride", _i64), ("v_head_stride", _i64),
                 ("H", _i32), ("Hkv", _i32), ("dim", _i32), ("vdim", _i32), ("scale", _f32), ("window", _i32),
-                ("sink", _vp), ("gate", _vp), ("ldg", _i64), ("out", _vp), ("ldo", _i64)]
+                ("sink", _vp), ("gate", _vp), ("ldg", _i64), ("out", _vp), ("ldo", _i64),
+                ("block", _i32), ("gate_cols", _i32), ("slots", _i32), ("k_slot_stride", _i64), ("v_slot_stride", _i64)]
 
 
 class AttnLatentArgs(C.Structure):
@@ -154,6 +156,27 @@ class AttnLatentArgs(C.Structure):
                 ("cache", _vp), ("slot_stride", _i64), ("row_stride", _i64),
                 ("H", _i32), ("dim", _i32), ("vdim", _i32), ("scale", _f32), ("window", _i32),
                 ("sink", _vp), ("gate", _vp), ("ldg", _i64), ("out", _vp), ("ldo", _i64), ("n_splits", _i32), ("part", _vp)]
+
+
+class AttnRowsArgs(C.Structure):
+    """``pcb_attn_rows_args`` (field for field)."""
+    _fields_ = [("struct_bytes", C.c_uint32), ("dtype", _i32),
+                ("q", _vp), ("ldq", _i64), ("tiles", _vp), ("n_rows", _i32),
+                ("k", _vp), ("k_slot_stride", _i64), ("k_head_stride", _i64), ("k_row_stride", _i64),
+                ("v", _vp), ("v_slot_stride", _i64), ("v_head_stride", _i64), ("v_row_stride", _i64),
+                ("H", _i32), ("Hkv", _i32), ("dim", _i32), ("vdim", _i32), ("scale", _f32), ("window", _i32), ("block", _i32),
+                ("sink", _vp), ("gate", _vp), ("ldg", _i64), ("gate_per_head", _i32), ("out", _vp), ("ldo", _i64), ("n_splits", _i32), ("part", _vp)]
+
+
+class RecArgs(C.Structure):
+    """``pcb_rec_args`` (field for field)."""
+    _fields_ = [("struct_bytes", C.c_uint32), ("dtype", _i32),
+                ("q", _vp), ("k", _vp), ("v", _vp), ("ldq", _i64), ("ldk", _i64), ("ldv", _i64),
+                ("unit_norm", _i32), ("unit_eps", _f32), ("rot", _vp), ("rot_dims", _i32), ("q_scale", _f32), ("k_scale", _f32),
+                ("decay", _vp), ("ld", _vp), ("ldld", _i64), ("ld_coef", _vp), ("ld_softplus", _i32), ("beta", _vp), ("ldbeta", _i64),
+                ("reqs", _vp), ("n_reqs", _i32), ("chunks", _vp), ("chunk0", _vp), ("n_chunks", _i32), ("state", _vp), ("slot_stride", _i64),
+                ("H", _i32), ("Hk", _i32), ("dim", _i32), ("vdim", _i32), ("scratch", _vp), ("scratch_floats", _i64), ("out", _vp), ("ldo", _i64),
+                ("gain", _vp), ("eps", _f32), ("gate", _vp), ("ldg", _i64), ("y", _vp), ("ldy", _i64)]
 
 
 # name -> (restype, argtypes); mirrors include/promptcache_blocks.h one to one
@@ -188,6 +211,13 @@ SIGNATURES = {
     "pcb_gla": (C.c_int, [C.POINTER(GlaArgs), _vp]),
     "pcb_attn_prompt": (C.c_int, [C.POINTER(AttnPromptArgs), _vp]),
     "pcb_attn_latent": (C.c_int, [C.POINTER(AttnLatentArgs), _vp]),
+    "pcb_attn_rows": (C.c_int, [C.POINTER(AttnRowsArgs), _vp]),
+    "pcb_rot_table": (C.c_int, [_vp, _vp, _f32, _vp, _i32, _i32, _vp]),
+    "pcb_conv_step": (C.c_int, [_vp, _i64, _vp, _vp, _i32, _i32, _vp, _i32, _vp, _i64, _vp, _i64, _i32, _i32, _vp]),
+    "pcb_rec_scratch": (C.c_int64, [_i32, _i32, _i32]),
+    "pcb_rec_prompt": (C.c_int, [C.POINTER(RecArgs), _vp]),
+    "pcb_rec_step_fits": (C.c_int32, [_i32, _i32]),
+    "pcb_rec_step": (C.c_int, [C.POINTER(RecArgs), _vp]),
 }
 
 
@@ -462,14 +492,15 @@ def hyper_norm(streams: torch.Tensor, *, y=None, mix=None, out_w=None, in_w=None
 
 def gated_norm(x: torch.Tensor, gain: Optional[torch.Tensor], gate: Optional[torch.Tensor], ldg: int, out: torch.Tensor, eps: float,
                n_rows: int, group: int = 0, gate_first: bool = False, skip: Optional[torch.Tensor] = None, lds: int = 0,
-               skip_w: Optional[torch.Tensor] = None, skip_group: int = 0) -> None:
+               skip_w: Optional[torch.Tensor] = None, skip_group: int = 0, ldo: Optional[int] = None) -> None:
     """``x`` fp32 [rows, cols]; ``gate`` E, a column block (row stride ``ldg``) of a wider matrix; ``out`` E [rows, cols].
     ``group`` > 0: a norm per run of that many columns (per head) instead of one over the row.  ``skip`` (E rows of stride
     ``lds``) with ``skip_w`` (fp32, one weight per ``skip_group`` columns): x + skip_w * skip stands for x.  ``gate_first``: the
-    gate is applied before the norm."""
+    gate is applied before the norm.  ``ldo``: row stride of ``out`` when it is a column block of a wider matrix."""
     _want(x, torch.float32, "gated_norm x"); _want(gain, torch.float32, "gated_norm gain"); _want(skip_w, torch.float32, "gated_norm skip_w")
     cols = x.shape[-1]
-    assert out.is_contiguous() and out.shape[-1] == cols and x.shape[0] >= n_rows and out.shape[0] >= n_rows
+    assert x.shape[0] >= n_rows and out.shape[0] >= n_rows
+    assert (out.is_contiguous() and out.shape[-1] == cols) if ldo is None else (ldo >= cols and _reach(out) >= (n_rows - 1) * ldo + cols)
     assert gain is None or gain.numel() == cols
     if gate is not None:
         assert gate.dtype == out.dtype and gate.is_cuda and ldg >= cols
@@ -477,7 +508,7 @@ def gated_norm(x: torch.Tensor, gain: Optional[torch.Tensor], gate: Optional[tor
         assert skip.dtype == out.dtype and skip.is_cuda and lds >= cols and skip_group > 0 and cols % skip_group == 0
         assert skip_w is not None and skip_w.numel() == cols // skip_group
     assert group == 0 or cols % group == 0
-    check(load().pcb_gated_norm(_p(x), cols, _p(gain), _p(gate), ldg, _p(out), cols, _code(out), float(eps), n_rows, cols, int(group),
+    check(load().pcb_gated_norm(_p(x), cols, _p(gain), _p(gate), ldg, _p(out), cols if ldo is None else ldo, _code(out), float(eps), n_rows, cols, int(group),
                                 int(gate_first), _p(skip), int(lds), _p(skip_w), int(skip_group), _stream()), "pcb_gated_norm")
 
 
@@ -608,19 +639,20 @@ def state_chain(local: torch.Tensor, start: torch.Tensor, state: torch.Tensor, c
 # ---- sublayers between two norms, per-head preparation, matrix memories ----------------------------------------------------------
 def post_norm(x: torch.Tensor, *, y=None, gate=None, ldg: int = 0, post_gain=None, gain=None, out=None, x_out=None, rows=None,
               eps: float = 1e-6, n_rows: Optional[int] = None, y_scale: float = 1.0, layer_norm: bool = False, bias=None,
-              pair=None, pair_weight=None, pair_top: int = 0, ldo: int = 0) -> None:
+              pair=None, pair_weight=None, pair_top: int = 0, ldo: int = 0, add=None) -> None:
     """``x`` fp32 [T, W] (the residual).  With ``y`` (fp32 [T, W]): x += norm(y * gate) * post_gain (``gate`` E rows of stride
     ``ldg``; without ``post_gain`` the gated y is added as it is).  With ``out`` (E): out = norm(x) * gain, for the rows ``rows``
     only if given (then x itself is not rewritten); ``x_out`` fp32 receives those rows of x.  ``y_scale``: the factor on what is
     added to x; ``layer_norm``: out = (x - mean) / sqrt(variance + eps) * gain + bias instead of the RMS form.
     ``pair`` fp32 [T * pair_top, W] with ``pair_weight``: sum_k weight * pair row joins ``y`` (or stands for it).  Without ``gain``,
-    ``out`` = x as E; ``ldo``: its row stride when it is a column block of a wider matrix."""
+    ``out`` = x as E; ``ldo``: its row stride when it is a column block of a wider matrix.  ``add`` fp32 [T, W]: x += add as well."""
     _want(x, torch.float32, "post_norm x"); _want(bias, torch.float32, "post_norm bias")
     assert bias is None or (layer_norm and bias.numel() == x.shape[-1])
     T, W = x.shape
     n = (rows.numel() if rows is not None else T) if n_rows is None else n_rows
-    for t, nm in ((y, "y"), (post_gain, "post_gain"), (gain, "gain"), (x_out, "x_out")):
+    for t, nm in ((y, "y"), (post_gain, "post_gain"), (gain, "gain"), (x_out, "x_out"), (add, "add")):
         _want(t, torch.float32, "post_norm " + nm)
+    assert add is None or (add.shape[-1] == W and add.shape[0] >= (T if rows is not None else n))
     assert rows is not None or n <= T
     if y is not None:
         assert y.shape[-1] == W and y.shape[0] >= (T if rows is not None else n)
@@ -641,7 +673,7 @@ def post_norm(x: torch.Tensor, *, y=None, gate=None, ldg: int = 0, post_gain=Non
     if rows is not None:
         _want(rows, torch.int32, "post_norm rows")
     a = PostNormArgs(C.sizeof(PostNormArgs), code, _p(x), _p(y), _p(gate), ldg, _p(post_gain), _p(gain), _p(out), _p(x_out), _p(rows),
-                     float(eps), n, W, float(y_scale), int(layer_norm), _p(bias), _p(pair), _p(pair_weight), pair_top, ldo)
+                     float(eps), n, W, float(y_scale), int(layer_norm), _p(bias), _p(pair), _p(pair_weight), pair_top, ldo, _p(add))
     check(load().pcb_post_norm(C.byref(a), _stream()), "pcb_post_norm")
 
 
@@ -667,14 +699,18 @@ def head_seg(src: torch.Tensor, ld_src: int, heads: int, head_dim: int, dst: tor
 
 
 def head_prep(segs, n_rows: int, dtype, *, pos: Optional[torch.Tensor] = None, freqs: Optional[torch.Tensor] = None, rot_mag: float = 1.0,
-              eps: float = 1e-6, rot_half: bool = False) -> None:
+              eps: float = 1e-6, rot_half: bool = False, table: Optional[torch.Tensor] = None) -> None:
     """``segs``: one to four ``head_seg`` records; ``pos`` int32 [rows]; ``freqs`` float64 [rot_dims / 2];
-    ``rot_half``: column i turns with column i + rot_dims / 2 instead of its neighbour."""
+    ``rot_half``: column i turns with column i + rot_dims / 2 instead of its neighbour; ``table``: fp32 rows of ``rot_table`` that stand
+    for ``pos``, ``freqs`` and ``rot_mag``."""
     _want(pos, torch.int32, "head_prep pos"); _want(freqs, torch.float64, "head_prep freqs")
     assert 1 <= len(segs) <= 4
     rot = {s.rot_dims for s in segs if s.rot_dims}
-    assert len(rot) <= 1 and (not rot or (pos is not None and freqs is not None and pos.numel() >= n_rows and 2 * freqs.numel() == rot.pop()))
+    _want(table, torch.float32, "head_prep table")
+    assert table is None or not rot or table.numel() >= n_rows * max(rot)
+    assert len(rot) <= 1 and (not rot or table is not None or (pos is not None and freqs is not None and pos.numel() >= n_rows and 2 * freqs.numel() == rot.pop()))
     a = HeadPrepArgs(C.sizeof(HeadPrepArgs), DTYPES[dtype], n_rows, len(segs), _p(pos), _p(freqs), float(rot_mag), float(eps), int(rot_half))
+    a.table = _p(table)
     for i, sg in enumerate(segs):
         a.seg[i] = sg
     check(load().pcb_head_prep(C.byref(a), _stream()), "pcb_head_prep")
@@ -747,18 +783,23 @@ def gla(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, ld: torch.Tensor, lds
 # ---- attention over rows rebuilt from a latent (prompts) and over the latent itself (decoding) -----------------------------------------
 def attn_prompt(q: torch.Tensor, tiles: torch.Tensor, n_tiles: int, tile_rows: int, k: torch.Tensor, k_strides, v: torch.Tensor, v_strides,
                 H: int, Hkv: int, dim: int, vdim: int, scale: float, out: torch.Tensor, *, ldo: int, ldq: Optional[int] = None, k_tail=None,
-                tail_row_stride: int = 0, tail_rows=None, tail_dim: int = 0, window: int = 0, sink=None, gate=None, ldg: int = 0) -> None:
-    """``k_strides`` / ``v_strides``: (row, head) strides in elements of the key and value rows; ``tail_rows``: int32 row of ``k_tail`` per
-    key row; ``gate``: E, one number per row and head."""
+                tail_row_stride: int = 0, tail_rows=None, tail_dim: int = 0, window: int = 0, sink=None, gate=None, ldg: int = 0,
+                block: int = 0, gate_cols: bool = False) -> None:
+    """``k_strides`` / ``v_strides``: (row, head) strides in elements of the key and value rows -- or (row, head, slot) strides: the tiles
+    then name slots; ``tail_rows``: int32 row of ``k_tail`` per key row; ``gate``: E, one number per row and head (or, ``gate_cols``, per
+    element); ``block`` > 0: a key is seen inside the query's own block of that many positions only."""
     _want(tiles, torch.int32, "attn_prompt tiles"); _want(sink, torch.float32, "attn_prompt sink"); _want(tail_rows, torch.int32, "attn_prompt tail_rows")
     assert q.dtype == k.dtype == v.dtype == out.dtype and q.is_cuda and k.is_cuda and v.is_cuda and out.is_cuda
     ldq = q.shape[-1] if ldq is None else ldq
     assert tiles.numel() >= 4 * n_tiles and ldq >= H * dim and ldo >= H * vdim and (sink is None or sink.numel() >= H)
     assert tail_dim == 0 or (k_tail is not None and k_tail.dtype == q.dtype and tail_row_stride >= tail_dim)
-    assert gate is None or (gate.dtype == q.dtype and ldg >= H)
+    assert gate is None or (gate.dtype == q.dtype and ldg >= (H * vdim if gate_cols else H))
+    slots = len(k_strides) == 3
+    assert len(v_strides) == len(k_strides) and not (slots and tail_dim)
     a = AttnPromptArgs(C.sizeof(AttnPromptArgs), _code(q), _p(q), ldq, _p(tiles), n_tiles, tile_rows, _p(k), k_strides[0], k_strides[1],
                        _p(k_tail), tail_row_stride, _p(tail_rows), tail_dim, _p(v), v_strides[0], v_strides[1], H, Hkv, dim, vdim, float(scale),
-                       int(window), _p(sink), _p(gate), ldg, _p(out), ldo)
+                       int(window), _p(sink), _p(gate), ldg, _p(out), ldo, int(block), int(gate_cols), int(slots), k_strides[2] if slots else 0,
+                       v_strides[2] if slots else 0)
     check(load().pcb_attn_prompt(C.byref(a), _stream()), "pcb_attn_prompt")
 
 
@@ -775,3 +816,90 @@ def attn_latent(q: torch.Tensor, tiles: torch.Tensor, n_rows: int, cache: torch.
     a = AttnLatentArgs(C.sizeof(AttnLatentArgs), _code(q), _p(q), q.shape[-1], _p(tiles), n_rows, _p(cache), slot_stride, row_stride, H, dim, vdim,
                        float(scale), int(window), _p(sink), _p(gate), ldg, _p(out), out.shape[-1], n_splits, _p(part))
     check(load().pcb_attn_latent(C.byref(a), _stream()), "pcb_attn_latent")
+
+
+# ---- decoding over cached rows, rotation tables, convolutions of one-token steps, matrix-state recurrences in chunks -------------------------
+def attn_rows(q: torch.Tensor, tiles: torch.Tensor, n_rows: int, k: torch.Tensor, k_strides, v: torch.Tensor, v_strides, H: int, Hkv: int, dim: int,
+              vdim: int, scale: float, out: torch.Tensor, *, ldo: int, ldq: Optional[int] = None, window: int = 0, block: int = 0, sink=None, gate=None,
+              ldg: int = 0, gate_per_head: bool = False, n_splits: int = 1, part=None) -> None:
+    """``tiles`` int32 {slot, position, 1, flat row} per row; ``k_strides`` / ``v_strides``: (slot, head, row) strides in elements of the cached
+    keys and values; ``gate``: E, element-wise or (``gate_per_head``) one number per row and head; ``part`` fp32 of
+    ``attn_softmax_part(rows, H, n_splits, vdim)`` floats when the keys are cut into runs."""
+    _want(tiles, torch.int32, "attn_rows tiles"); _want(sink, torch.float32, "attn_rows sink"); _want(part, torch.float32, "attn_rows part")
+    assert q.dtype == k.dtype == v.dtype == out.dtype and q.is_cuda and k.is_cuda and v.is_cuda and out.is_cuda
+    ldq = q.shape[-1] if ldq is None else ldq
+    assert tiles.numel() >= 4 * n_rows and ldq >= H * dim and ldo >= H * vdim and (sink is None or sink.numel() >= H)
+    assert gate is None or (gate.dtype == q.dtype and ldg >= (H if gate_per_head else H * vdim))
+    assert n_splits <= 1 or (part is not None and part.numel() >= attn_softmax_part(n_rows, H, n_splits, vdim))
+    a = AttnRowsArgs(C.sizeof(AttnRowsArgs), _code(q), _p(q), ldq, _p(tiles), n_rows, _p(k), *(int(x) for x in k_strides), _p(v),
+                     *(int(x) for x in v_strides), H, Hkv, dim, vdim, float(scale), int(window), int(block), _p(sink), _p(gate), ldg,
+                     int(gate_per_head), _p(out), ldo, n_splits, _p(part))
+    check(load().pcb_attn_rows(C.byref(a), _stream()), "pcb_attn_rows")
+
+
+def rot_table(pos: torch.Tensor, freqs: torch.Tensor, mag: float, out: torch.Tensor, n_rows: int) -> None:
+    """``out`` fp32 [rows, 2 * pairs]: mag * (cosines | sines) of pos * freqs (``pos`` int32, ``freqs`` float64 [pairs])."""
+    _want(pos, torch.int32, "rot_table pos"); _want(freqs, torch.float64, "rot_table freqs"); _want(out, torch.float32, "rot_table out")
+    assert pos.numel() >= n_rows and out.numel() >= 2 * n_rows * freqs.numel()
+    check(load().pcb_rot_table(_p(pos), _p(freqs), float(mag), _p(out), n_rows, freqs.numel(), _stream()), "pcb_rot_table")
+
+
+def conv_step(x: torch.Tensor, ldx: int, w: torch.Tensor, bias: Optional[torch.Tensor], silu: bool, reqs: torch.Tensor, n_reqs: int,
+              state: torch.Tensor, out: torch.Tensor) -> None:
+    """``causal_conv`` and ``conv_state_update`` at once, for a step of one token per request."""
+    C_, taps = w.shape
+    _want(reqs, torch.int32, "conv_step reqs")
+    assert x.dtype == w.dtype == out.dtype == state.dtype and out.is_contiguous() and out.shape[-1] == C_ and w.is_contiguous()
+    assert reqs.numel() >= 4 * n_reqs and tuple(state.shape[1:]) == (taps - 1, C_) and state.is_contiguous() and (bias is None or bias.numel() == C_)
+    check(load().pcb_conv_step(_p(x), ldx, _p(w), _p(bias), _code(x), int(silu), _p(reqs), n_reqs, _p(state), (taps - 1) * C_, _p(out), C_, C_, taps,
+                               _stream()), "pcb_conv_step")
+
+
+def rec_scratch(n_chunks: int, H: int, dim: int) -> int:
+    return int(load().pcb_rec_scratch(n_chunks, H, dim))
+
+
+def rec_step_fits(dim: int, vdim: int) -> bool:
+    return bool(load().pcb_rec_step_fits(dim, vdim))
+
+
+def _rec_args(q, k, v, lds_, reqs, n_reqs, state, H, Hk, dim, vdim, *, decay=None, ld=None, ldld=0, ld_coef=None, ld_softplus=False, beta=None,
+              ldbeta=0, unit_norm=False, unit_eps=1e-6, rot=None, rot_dims=0, q_scale=1.0, k_scale=1.0) -> RecArgs:
+    for t, nm in ((decay, "decay"), (ld_coef, "ld_coef"), (rot, "rot"), (state, "state")):
+        _want(t, torch.float32, "rec " + nm)
+    _want(reqs, torch.int32, "rec reqs")
+    assert q.dtype == k.dtype == v.dtype and q.is_cuda and reqs.numel() >= 4 * n_reqs and tuple(state.shape[-3:]) == (H, dim, vdim)
+    assert (decay is None) != (ld is None) and (decay is None or decay.numel() == H) and (ld_coef is None or ld_coef.numel() == H)
+    for t, st, n, nm in ((ld, ldld, H * dim, "ld"), (beta, ldbeta, H, "beta")):
+        assert t is None or (t.dtype == torch.float32 and t.is_cuda and st >= n), nm
+    a = RecArgs(C.sizeof(RecArgs), _code(q), _p(q), _p(k), _p(v), *(int(x) for x in lds_), int(unit_norm), float(unit_eps), _p(rot), rot_dims,
+                float(q_scale), float(k_scale), _p(decay), _p(ld), ldld, _p(ld_coef), int(ld_softplus), _p(beta), ldbeta, _p(reqs), n_reqs)
+    a.state, a.slot_stride, a.H, a.Hk, a.dim, a.vdim = _p(state), H * dim * vdim, H, Hk, dim, vdim
+    return a
+
+
+def rec_prompt(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, lds_, reqs: torch.Tensor, n_reqs: int, chunks: torch.Tensor, chunk0: torch.Tensor,
+               n_chunks: int, state: torch.Tensor, H: int, Hk: int, dim: int, vdim: int, scratch: torch.Tensor, out: torch.Tensor, **kw) -> None:
+    """``q``, ``k`` (``Hk`` heads), ``v`` (``H`` heads): E rows of strides ``lds_``; ``state`` fp32 [slots, H, dim, vdim]; ``chunks`` int32 {first
+    flat row, tokens, 0, 0} per 16 tokens, request r's from ``chunk0[r]`` on; ``out`` fp32 [rows, H * vdim].  Further arguments: ``decay``
+    fp32 [H], or ``ld`` (fp32 rows, stride ``ldld``) with ``ld_coef`` / ``ld_softplus``; ``beta`` (fp32 rows, stride ``ldbeta``): the delta
+    rule; ``unit_norm`` / ``unit_eps``; ``rot`` / ``rot_dims``: a ``rot_table``; ``q_scale``, ``k_scale``."""
+    _want(chunks, torch.int32, "rec chunks"); _want(chunk0, torch.int32, "rec chunk0"); _want(scratch, torch.float32, "rec scratch")
+    _want(out, torch.float32, "rec out")
+    assert chunks.numel() >= 4 * n_chunks and chunk0.numel() >= n_reqs and out.shape[-1] == H * vdim
+    a = _rec_args(q, k, v, lds_, reqs, n_reqs, state, H, Hk, dim, vdim, **kw)
+    a.chunks, a.chunk0, a.n_chunks = _p(chunks), _p(chunk0), n_chunks
+    a.scratch, a.scratch_floats, a.out, a.ldo = _p(scratch), scratch.numel(), _p(out), H * vdim
+    check(load().pcb_rec_prompt(C.byref(a), _stream()), "pcb_rec_prompt")
+
+
+def rec_step(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, lds_, reqs: torch.Tensor, n_reqs: int, state: torch.Tensor, H: int, Hk: int, dim: int,
+             vdim: int, y: torch.Tensor, ldy: int, *, eps: float, gain=None, gate=None, ldg: int = 0, **kw) -> None:
+    """The same recurrence for a step of one token per request, on to the head's output norm (``gain`` fp32 [vdim]) and ``gate`` (E rows):
+    ``y`` E rows of stride ``ldy``."""
+    _want(gain, torch.float32, "rec gain")
+    assert y.dtype == q.dtype and y.is_cuda and ldy >= H * vdim and (gain is None or gain.numel() == vdim)
+    assert gate is None or (gate.dtype == q.dtype and ldg >= H * vdim)
+    a = _rec_args(q, k, v, lds_, reqs, n_reqs, state, H, Hk, dim, vdim, **kw)
+    a.gain, a.eps, a.gate, a.ldg, a.y, a.ldy = _p(gain), float(eps), _p(gate), ldg, _p(y), ldy
+    check(load().pcb_rec_step(C.byref(a), _stream()), "pcb_rec_step")
