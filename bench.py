@@ -862,6 +862,51 @@ def run_pikadra(args):
     print(json.dumps(out))
 
 
+def run_venitar(args):
+    """Throughput of the Venitar stack beside the Bepepel stack (the closest existing model: the same building-block library, bf16
+    tensors, an fp32 residual, a matrix-state recurrence with a decay per key channel, an attention and a recurrence side by side) and
+    beside the Fivesun stack's block attention, at equal width, heads and depth, with feed-forwards of equal work (Bepepel: 2 of 16
+    experts of width / 2 plus a shared one, 4.5 w^2 per token; Fivesun: a gated unit of 2 w, 6 w^2; Venitar: two matrices of 2.25 w,
+    `attention` 3 w).
+
+    Per size: one prompt of 2048 tokens (tokens/s of the prefill), then decoding at a context of 2048 with 1 and 8 requests.
+    `retention` / `parallel` / `attention` = four layers of that mixer alone, which is what prices each mixer's kernels (beside
+    Bepepel's `gla` and `parallel` and Fivesun's `attention`); `mixed` = retention, parallel, attention, retention; `loop` = `mixed` with
+    the middle two layers run twice (six layer runs).  The window and the blocks have 1024 positions.  Random weights, synthetic tokens."""
+    import torch
+    import __graft_entry__ as ge
+    ge.build()
+    from promptcache_amd.model import Bepepel, Fivesun, Venitar
+    from promptcache_amd.model.config import BepepelShape, FivesunShape, VenitarShape
+    dev = "cuda:0"
+    torch.cuda.set_device(0)
+    sizes = {"2k": dict(width=2048, heads=16, kv=4), "4k": dict(width=4096, heads=32, kv=8)}
+    L, V, T, steps, warm = 4, 32000, 2048, max(4, min(args.steps, 20)), max(1, min(args.warmup, 3))
+    g = torch.Generator().manual_seed(0)
+    out = {"metric": "venitar_throughput", "unit": "tokens/s", "dtype": "bf16", "data": "synthetic", "layers": L, "prompt": T, "sizes": {}}
+    mixed = ["retention", "parallel", "attention", "retention"]
+    patterns = {"mixed": mixed, "loop": mixed, "retention": ["retention"] * L, "parallel": ["parallel"] * L, "attention": ["attention"] * L}
+    for key in args.venitar_sizes.split(","):
+        c = sizes[key]
+        w, h = c["width"], c["heads"]
+        row = {"width": w, "heads": h}
+        for pk in (("gla", "parallel") if args.venitar_baseline else ()):
+            bp = BepepelShape.uniform(V, w, [pk] * L, h, c["kv"], w // h, experts=16, top=2, expert_ff=w // 2, window=1024, keep_first=4,
+                                      name=f"bepepel-{key}-{pk}")
+            row["bepepel_" + pk] = slot_model_case(Bepepel(shape=bp, random_init=True, seed=0, device=dev), V, T, steps, warm, g)
+        if args.venitar_baseline:
+            fs = FivesunShape.uniform(V, w, ["attention"] * L, h, c["kv"], w // h, 2 * w, chunk=1024, window=1024, kv_rank=192, rot_dim=64,
+                                      name=f"fivesun-{key}-attention")
+            row["fivesun_attention"] = slot_model_case(Fivesun(shape=fs, random_init=True, seed=0, device=dev), V, T, steps, warm, g)
+        for pk in args.venitar_patterns.split(","):
+            shape = VenitarShape.uniform(V, w, patterns[pk], h, c["kv"], w // h, 3 * w if pk == "attention" else 9 * w // 4, block=1024, window=1024,
+                                         loop=(1, 3, 2) if pk == "loop" else None, name=f"venitar-{key}-{pk}")
+            row["venitar_" + pk] = slot_model_case(Venitar(shape=shape, random_init=True, seed=0, device=dev), V, T, steps, warm, g)
+        out["sizes"][key] = row
+        print(json.dumps({key: row}), file=sys.stderr, flush=True)
+    print(json.dumps(out))
+
+
 def run_kazolorn(args):
     """Throughput of the Kazolorn stack beside the MPT stack at equal width, heads, depth and feed-forward width.
 
@@ -965,6 +1010,12 @@ def main():
                          "real models (random weights), beside the Kazolorn stack (the closest existing model) at equal size")
     ap.add_argument("--dibizen-sizes", default="2k,4k", help="--dibizen: which sizes (2k, 4k)")
     ap.add_argument("--dibizen-patterns", default="mixed,attention,lightning,mamba1", help="--dibizen: which layer patterns")
+    ap.add_argument("--venitar", action="store_true",
+                    help="instead of the default workload: prefill / decode throughput of the Venitar design at layer sizes of "
+                         "real models, beside the Bepepel and Fivesun stacks at equal size")
+    ap.add_argument("--venitar-sizes", default="2k,4k", help="--venitar: which sizes (2k, 4k)")
+    ap.add_argument("--venitar-patterns", default="mixed,retention,parallel,attention,loop", help="--venitar: which stacks")
+    ap.add_argument("--venitar-baseline", type=int, default=1, help="--venitar: 0 leaves the other stacks out (kernel profiles of Venitar alone)")
     ap.add_argument("--pikadra", action="store_true",
                     help="instead of the default workload: prefill / decode throughput of the Pikadra design at layer sizes of "
                          "real models, beside the Fivesun stack's latent attention at equal size")
@@ -992,6 +1043,9 @@ def main():
         return
     if args.dibizen:
         run_dibizen(args)
+        return
+    if args.venitar:
+        run_venitar(args)
         return
     if args.pikadra:
         run_pikadra(args)

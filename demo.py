@@ -12,6 +12,7 @@ cache and once with ``no_cache=True``, printing the two timed intervals of each 
     python demo.py --model fivesun                   # the Fivesun design (attention / latent attention / mlstm layers), likewise
     python demo.py --model bepepel                   # the Bepepel design (gla / parallel attention + state-space layers), likewise
     python demo.py --model pikadra                   # the Pikadra design (latent attention beside experts, a loop of layers), likewise
+    python demo.py --model venitar                   # the Venitar design (retention, block attention, windowed attention + gated delta rule), likewise
 
 There is no network on the build / bench machines, so without a checkpoint directory the adapters use seeded random
 weights at the named shape and the deterministic stand-in tokenizer: the text is noise, the timings are real.
@@ -24,8 +25,8 @@ ROOT = os.path.dirname(os.path.abspath(__file__))
 sys.path.insert(0, os.path.join(ROOT, "prompt-cache_amd"))
 
 from promptcache_amd import CacheEngine, GenerationEngine, GenerationParameters, Prompt, read_file, synth  # noqa: E402
-from promptcache_amd.model import Bepepel, CodeLlama, Dibizen, Falcon, Fivesun, Kazolorn, Llama2, Mpt, Pikadra, load_language_model  # noqa: E402
-from promptcache_amd.model.config import BepepelShape, DibizenShape, FivesunShape, KazolornShape, PikadraShape  # noqa: E402
+from promptcache_amd.model import Bepepel, CodeLlama, Dibizen, Falcon, Fivesun, Kazolorn, Llama2, Mpt, Pikadra, Venitar, load_language_model  # noqa: E402
+from promptcache_amd.model.config import BepepelShape, DibizenShape, FivesunShape, KazolornShape, PikadraShape, VenitarShape  # noqa: E402
 
 ADAPTERS = {"llama": (Llama2, "llama2-7b"), "codellama": (CodeLlama, "codellama-7b"), "falcon": (Falcon, "falcon-7b"),
             "mpt": (Mpt, "mpt-7b")}
@@ -53,7 +54,7 @@ def kazolorn_demo(lm, a):
 
 def main():
     ap = argparse.ArgumentParser()
-    ap.add_argument("--model", default="llama", help="llama | codellama | falcon | mpt | kazolorn | dibizen | fivesun | bepepel | pikadra | <checkpoint directory>")
+    ap.add_argument("--model", default="llama", help="llama | codellama | falcon | mpt | kazolorn | dibizen | fivesun | bepepel | pikadra | venitar | <checkpoint directory>")
     ap.add_argument("--schema", help="PML schema file (default: a synthetic game-like schema, 7 modules)")
     ap.add_argument("--prompt-file", help="PML prompt file referencing the schema")
     ap.add_argument("--max-ctx", type=int, default=5000)
@@ -79,10 +80,13 @@ def main():
     elif a.model == "pikadra":
         lm = Pikadra(shape=PikadraShape.uniform(32000, 1024, 4, 8, 128, 64, 256, 384, experts=8, top=2, expert_ff=512, shared_ff=512,
                                                 loop=(1, 3, 2)), random_init=True)
+    elif a.model == "venitar":
+        lm = Venitar(shape=VenitarShape.uniform(32000, 1024, ["retention", "parallel", "attention", "retention"], 8, 2, 128, 2048, block=512,
+                                                window=512, loop=(1, 3, 2)), random_init=True)
     else:
         cls, shape = ADAPTERS[a.model]
         lm = cls(shape, random_init=True)
-    if isinstance(lm, (Kazolorn, Dibizen, Fivesun, Bepepel, Pikadra)):
+    if isinstance(lm, (Kazolorn, Dibizen, Fivesun, Bepepel, Pikadra, Venitar)):
         kazolorn_demo(lm, a)
         return
     preproc = [lm.get_formatter()]

@@ -2,7 +2,7 @@
 // without a gain), a blend with another layer's values, rotary positions on neighbouring column pairs or on halves, and the store into a row
 // matrix or a slot's cache (row by row or column by column).  Up to four segments (queries, keys, values, ...) per launch.
 //
-// One workgroup per (row, segment).  The turn of every column pair depends on the row's position only, so the workgroup first
+// One workgroup per (row, segment), or several that share the heads when rows are few.  The turn of every column pair depends on the row's position only, so the workgroup first
 // fills a cos / sin table in LDS -- the angle is the float64 product position x frequency, reduced by float64 sincos, so a
 // position in the thousands costs no bits of the angle -- and its waves then take the heads in turn: one pass for the sum of
 // squares, one that norms, blends, turns and stores.  A lane owns the two columns of a pair, so a rotation never crosses lanes
@@ -24,7 +24,7 @@ __device__ __forceinline__ void prep_heads(const pcb_head_prep_args& a, const pc
     const int first = LONE ? (int)threadIdx.x : lane;
     constexpr int STEP = LONE ? 256 : 64;
     const float lam = s.blend ? s.blend[0] : 0.0f;
-    for (int h = LONE ? 0 : wave; h < s.heads; h += 4) {
+    for (int h = LONE ? 0 : wave + 4 * (int)blockIdx.z; h < s.heads; h += 4 * (int)gridDim.z) {
         const E* x = (const E*)s.src + row * s.ld_src + (int64_t)h * s.src_head_stride;
         float inv = 1.0f;
         if (s.norm) {
@@ -113,6 +113,7 @@ __global__ __launch_bounds__(256) void head_prep_kernel(pcb_head_prep_args a) {
         }
         __syncthreads();
     }
+    if (s.heads == 1 && blockIdx.z > 0) return;
     if (s.heads == 1)
         prep_heads<E, true>(a, s, row, cs, sn, red);
     else
@@ -161,7 +162,10 @@ PCB_EXPORT int pcb_head_prep(const pcb_head_prep_args* a, void* stream) {
     }
     if (a->n_rows == 0) return PCB_OK;
     PCB_REQUIRE(rot == 0 || a->table || (a->pos && a->freqs), PCB_ERR_ARG, "pcb_head_prep: a rotation needs positions and frequencies");
-    const dim3 grid(a->n_rows, a->n_segs);
+    // (few rows: a row's heads are spread over workgroups, so that a wave has one)
+    int most = 1;
+    for (int i = 0; i < a->n_segs; ++i) most = a->seg[i].heads > most ? a->seg[i].heads : most;
+    const dim3 grid(a->n_rows, a->n_segs, a->n_rows <= 64 ? pcb_ceil_div(most < 64 ? most : 64, 4) : 1);
     if (a->dtype == PCB_BF16)
         hipLaunchKernelGGL(head_prep_kernel<pcb::bf16_t>, grid, dim3(256), 0, (hipStream_t)stream, *a);
     else

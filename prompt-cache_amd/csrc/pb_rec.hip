@@ -27,7 +27,21 @@ __device__ __forceinline__ float exp2_(float x) { return __builtin_amdgcn_exp2f(
 // decay^n for a small non-negative integer n
 __device__ __forceinline__ float decay_pow(float log2_decay, int n) { return n <= 0 ? 1.0f : exp2f((float)n * log2_decay); }
 __device__ __forceinline__ float log2_of(float decay) { return decay > 0.0f ? log2f(decay) : -__builtin_inff(); }
-__device__ __forceinline__ float softplus(float z) { return z > 20.0f ? z : log1pf(expf(z)); }
+// ln(1 + e^z) = max(z, 0) + ln(1 + x), x = e^-|z| <= 1, and ln(1 + x) = 2 artanh(y), y = x / (2 + x) <= 1/3, by artanh's odd power series
+__device__ __forceinline__ float softplus(float z) {
+    const float x = __builtin_amdgcn_exp2f(-fabsf(z) * 1.44269504088896f);
+    const float y = x * __builtin_amdgcn_rcpf(2.0f + x), y2 = y * y;
+    float p = 1.0f / 17.0f;
+    p = p * y2 + 1.0f / 15.0f;
+    p = p * y2 + 1.0f / 13.0f;
+    p = p * y2 + 1.0f / 11.0f;
+    p = p * y2 + 1.0f / 9.0f;
+    p = p * y2 + 1.0f / 7.0f;
+    p = p * y2 + 1.0f / 5.0f;
+    p = p * y2 + 1.0f / 3.0f;
+    p = p * y2 + 1.0f;
+    return fmaxf(z, 0.0f) + 2.0f * y * p;
+}
 __device__ __forceinline__ float sigmoid(float z) { return 1.0f / (1.0f + expf(-z)); }
 
 // the log decay (in units of ln 2) a row of `ld` stands for
@@ -35,9 +49,10 @@ __device__ __forceinline__ float log2_decay(const pcb_rec_args& a, float x, floa
     return (a.ld_softplus ? softplus(x) : x) * coef * LOG2E;
 }
 
-// floats of one (chunk, head) record: Q' | K^ | T K~ as fragments, the end decays, M and T
-__host__ __device__ inline int rec_tiles(int dim) { return (dim + 15) / 16; }
-__host__ __device__ inline int64_t rec_record(int dim) { return (int64_t)rec_tiles(dim) * (3 * 256 + 16) + 512; }
+// one (chunk, head) record of `tiles` 16-column tiles (the key size filled up to 64, 128 or 256 columns): Q~ - M K~, K^ and -T K~ as
+// fragments, the end decays, M and T; and its floats
+__host__ __device__ constexpr int rec_columns(int dim) { return dim <= 64 ? 64 : dim <= 128 ? 128 : 256; }
+__host__ __device__ constexpr int rec_record(int tiles) { return tiles * (3 * 256 + 16) + 512; }
 
 // DM: key columns the workgroup holds (>= dim); DELTA: with the correction; ROWS: decays per key channel and token
 template <typename E, int DM, bool DELTA, bool ROWS>
@@ -50,8 +65,8 @@ __global__ __launch_bounds__(256) void rec_prep_kernel(pcb_rec_args a) {
     const int64_t row0 = ck[0];
     const int n = ck[1];
     const int t = tid >> 4, s = tid & 15;                  // a token and one of 16 threads that share it
-    float* rec = a.scratch + ((int64_t)blockIdx.y * a.H + h) * rec_record(D);
-    const int NT = rec_tiles(D);
+    constexpr int NT = DM / 16;
+    float* rec = a.scratch + ((int64_t)blockIdx.y * a.H + h) * rec_record(NT);
     float* rq = rec;
     float* rk = rq + NT * 256;
     float* rw = rk + NT * 256;
@@ -89,18 +104,28 @@ __global__ __launch_bounds__(256) void rec_prep_kernel(pcb_rec_args a) {
             *reinterpret_cast<f4*>(&Ks[t][4 * s + 64 * i]) = f4{kv[i][0] * fk, kv[i][1] * fk, kv[i][2] * fk, kv[i][3] * fk};
         }
     }
-    if (ROWS && tid < DM) {
-        // running sums of the log decays, a thread per key channel (tokens past the end and columns past dim: no decay)
-        float l[CT];
+    if (ROWS) {
+        // log decays (tokens past the end and columns past dim: none), then their running sums, a thread per key channel
         const float coef = a.ld_coef ? a.ld_coef[h] : 1.0f;
-        const float* ld = a.ld + row0 * a.ldld + (int64_t)h * D + tid;
+        const float* ld = a.ld + (row0 + t) * a.ldld + (int64_t)h * D;
+        const bool vec = D % 4 == 0 && a.ldld % 4 == 0 && (uintptr_t)a.ld % 16 == 0;
 #pragma unroll
-        for (int i = 0; i < CT; ++i) l[i] = (i < n && tid < D) ? ld[(int64_t)i * a.ldld] : 0.0f;
-        float cum = 0.0f;
+        for (int i = 0; i < DM / 64; ++i) {
+            const int d0 = 4 * s + 64 * i;
+            float l[4];
+            load4(ld + d0, vec, t < n ? D - d0 : 0, l);
+            f4 v;
 #pragma unroll
-        for (int i = 0; i < CT; ++i) {
-            if (i < n && tid < D) cum += log2_decay(a, l[i], coef);
-            Gs[ROWS ? i : 0][tid] = cum;
+            for (int e = 0; e < 4; ++e) v[e] = t < n && d0 + e < D ? log2_decay(a, l[e], coef) : 0.0f;
+            *reinterpret_cast<f4*>(&Gs[ROWS ? t : 0][d0]) = v;
+        }
+        __syncthreads();
+        if (tid < DM) {
+            float l[CT], cum = 0.0f;
+#pragma unroll
+            for (int i = 0; i < CT; ++i) l[i] = Gs[ROWS ? i : 0][tid];
+#pragma unroll
+            for (int i = 0; i < CT; ++i) Gs[ROWS ? i : 0][tid] = cum += l[i];
         }
     }
     __syncthreads();
@@ -116,19 +141,31 @@ __global__ __launch_bounds__(256) void rec_prep_kernel(pcb_rec_args a) {
         __syncthreads();
     }
 
-    // ---- A and B: a thread per pair of tokens (t, j = s)
-    const float beta = DELTA && t < n ? sigmoid(a.beta[(row0 + t) * a.ldbeta + h]) : 0.0f;
+    // ---- A and B.  The 120 pairs j < t take two threads each (neighbours, each half of the key columns), the 16 tokens with themselves
+    // one each (no decay, and A is not needed)
     {
-        const int j = s;
+        const bool self = tid >= 240;
+        int pt, pj, d_lo = 0, d_hi = DM;
+        if (self) {
+            pt = pj = tid - 240;
+        } else {
+            const int pr = tid >> 1;                       // pair t (t - 1) / 2 + j
+            pt = (int)((1.0f + sqrtf(1.0f + 8.0f * (float)pr)) * 0.5f);
+            if (pt * (pt - 1) / 2 > pr) --pt;
+            if (pt * (pt + 1) / 2 <= pr) ++pt;
+            pj = pr - pt * (pt - 1) / 2;
+            d_lo = tid & 1 ? DM / 2 : 0;
+            d_hi = d_lo + DM / 2;
+        }
         float pa = 0.0f, pb = 0.0f;
-        if (j <= t && t < n) {
+        if (pt < n) {
 #pragma unroll 4
-            for (int d = 0; d < DM; d += 4) {
-                const f4 kj = *reinterpret_cast<const f4*>(&Ks[j][d]), qt = *reinterpret_cast<const f4*>(&Qs[t][d]);
+            for (int d = d_lo; d < d_hi; d += 4) {
+                const f4 kj = *reinterpret_cast<const f4*>(&Ks[pj][d]), qt = *reinterpret_cast<const f4*>(&Qs[pt][d]);
                 f4 kt = kj, ex = kj;
-                if (DELTA) kt = *reinterpret_cast<const f4*>(&Ks[t][d]);
-                if (ROWS) {
-                    const f4 gt = *reinterpret_cast<const f4*>(&Gs[t][d]), gj = *reinterpret_cast<const f4*>(&Gs[j][d]);
+                if (DELTA) kt = *reinterpret_cast<const f4*>(&Ks[pt][d]);
+                if (ROWS && !self) {
+                    const f4 gt = *reinterpret_cast<const f4*>(&Gs[ROWS ? pt : 0][d]), gj = *reinterpret_cast<const f4*>(&Gs[ROWS ? pj : 0][d]);
 #pragma unroll
                     for (int e = 0; e < 4; ++e) ex[e] = kj[e] * exp2_(gt[e] - gj[e]);
                 }
@@ -138,31 +175,34 @@ __global__ __launch_bounds__(256) void rec_prep_kernel(pcb_rec_args a) {
                     if (DELTA) pa += kt[e] * ex[e];
                 }
             }
-            if (!ROWS) {
-                const float f = decay_pow(lg, t - j);
-                pa *= f;
-                pb *= f;
-            }
         }
-        Bs[t][j] = pb;
-        if (DELTA) As[t][j] = j < t ? beta * pa : 0.0f;
+        const float pa2 = pa + __shfl_xor(pa, 1, 64), pb2 = pb + __shfl_xor(pb, 1, 64);
+        if (self) {
+            Bs[pt][pt] = pb;
+            if (DELTA) {
+                const float beta = pt < n ? sigmoid(a.beta[(row0 + pt) * a.ldbeta + h]) : 0.0f;
+                As[pt][pt] = beta;                         // (the diagonal carries the step sizes)
+            }
+        } else if ((tid & 1) == 0) {
+            const float f = ROWS ? 1.0f : decay_pow(lg, pt - pj);
+            Bs[pt][pj] = pb2 * f;
+            Bs[pj][pt] = 0.0f;
+            if (DELTA) As[pt][pj] = pa2 * f;
+        }
     }
     __syncthreads();
 
     // ---- T by forward substitution, a thread per column; meanwhile the other waves turn q, k into Q~, K~ and store K^
-    if (DELTA) {
-        if (s == t) Ms[0][t] = beta;                       // (Ms waits for M: its first row carries the step sizes for a moment)
-        __syncthreads();
-        if (tid < CT) {
-            float x[CT];
+    if (DELTA && tid < CT) {
+        // (1 + diag(beta) A) T = diag(beta), row by row: T[r] = beta_r (e_r - sum over j < r of A[r][j] T[j])
+        float x[CT];
 #pragma unroll
-            for (int r = 0; r < CT; ++r) {
-                float v = r == tid ? Ms[0][tid] : 0.0f;
+        for (int r = 0; r < CT; ++r) {
+            float v = r == tid ? 1.0f : 0.0f;
 #pragma unroll
-                for (int j = 0; j < r; ++j) v -= As[r][j] * x[j];
-                x[r] = v;
-                Ts[r][tid] = v;
-            }
+            for (int j = 0; j < r; ++j) v -= As[r][j] * x[j];
+            x[r] = v * As[r][r];
+            Ts[r][tid] = x[r];
         }
     }
     for (int i = tid; i < 4 * DM; i += 256) {
@@ -188,8 +228,8 @@ __global__ __launch_bounds__(256) void rec_prep_kernel(pcb_rec_args a) {
             Ks[j][d] = kv * f_in;
             Qs[j][d] *= f_in;
         }
-        if (b < NT) *reinterpret_cast<f4*>(rk + (b * 64 + g * 16 + c) * 4) = kh;
-        if (g == 0 && b < NT) rd[d] = ROWS ? exp2_(g_end) : decay_pow(lg, n);
+        *reinterpret_cast<f4*>(rk + (b * 64 + g * 16 + c) * 4) = kh;
+        if (g == 0) rd[d] = ROWS ? exp2_(g_end) : decay_pow(lg, n);
     }
     __syncthreads();
 
@@ -230,18 +270,24 @@ __global__ __launch_bounds__(256) void rec_prep_kernel(pcb_rec_args a) {
     }
 }
 
-// NBW: 16-row tiles of S a wave holds (4 NBW tiles in all)
-template <typename E, int NBW, bool DELTA>
+// a value at a uniform address plus a lane's 32-bit byte offset
+template <typename T>
+__device__ __forceinline__ T at(const void* base, uint32_t bytes) {
+    return *reinterpret_cast<const T*>(reinterpret_cast<const char*>(base) + bytes);
+}
+
+// NBW: 16-row tiles of S a wave holds (4 NBW tiles in all); ROWS: the end decays come with the records (else decay[h]^tokens)
+template <typename E, int NBW, bool DELTA, bool ROWS>
 __global__ __launch_bounds__(256) void rec_scan_kernel(pcb_rec_args a) {
+    constexpr int NT = 4 * NBW, REC = rec_record(NT);
     __shared__ f4 red_u[DELTA ? 2 : 1][4][64];
     __shared__ float red_o[2][4][4][64];
-    const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6, g = lane >> 4, c = lane & 15;
+    const int lane = threadIdx.x & 63, w = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), g = lane >> 4, c = lane & 15;
     const int32_t* rq = a.reqs + 4 * blockIdx.z;
     const int slot = rq[0], pos0 = rq[1], count = rq[2];
     const int64_t row0 = rq[3];
     const int h = blockIdx.x, D = a.dim, vdim = a.vdim, vcol = blockIdx.y * 16 + c;
     const bool v_ok = vcol < vdim;
-    const int NT = rec_tiles(D);
     float* st = a.state + (int64_t)slot * a.slot_stride + (int64_t)h * D * vdim;
     f4 S[NBW];
 #pragma unroll
@@ -251,89 +297,128 @@ __global__ __launch_bounds__(256) void rec_scan_kernel(pcb_rec_args a) {
             const int d = 16 * (w * NBW + i) + 4 * g + r;
             S[i][r] = (pos0 > 0 && d < D && v_ok) ? st[(int64_t)d * vdim + vcol] : 0.0f;
         }
-    const int64_t stride = (int64_t)a.H * rec_record(D);
-    const float* rec = a.scratch + ((int64_t)a.chunk0[blockIdx.z] * a.H + h) * rec_record(D);
-    const E* V = (const E*)a.v + row0 * a.ldv + (int64_t)h * vdim + vcol;
-    constexpr int VN = DELTA ? 1 : 4;
-    f4 nq[NBW], nk[NBW], nw[DELTA ? NBW : 1], nd[NBW];
-    float nm, nt = 0.0f, nv[VN];
-    auto fetch = [&](int i) {                              // chunk i's operands
+    const int n_chunk = (count + CT - 1) / CT, n_last = count - CT * (n_chunk - 1);
+    const float lg = ROWS ? 0.0f : log2_of(a.decay[h]);
+    const float dec_full = ROWS ? 0.0f : decay_pow(lg, CT), dec_last = ROWS ? 0.0f : decay_pow(lg, n_last);
+    const int64_t stride = (int64_t)a.H * REC;
+    const float* rec = a.scratch + ((int64_t)a.chunk0[blockIdx.z] * a.H + h) * REC + w * NBW * 256;
+    const int w_dec = w * NBW * 16 - w * NBW * 256, w_mt = w * 64 - w * NBW * 256;
+    const E* V = (const E*)a.v + row0 * a.ldv + (int64_t)h * vdim;
+    // a ring of PF chunks' operands, read without branches: chunk i waits in slot i % PF and is replaced, part by part, by chunk i + PF once
+    // it has been used.  Chunks, tokens and columns past the end repeat the last one (their K^, M and T are zero, or nothing of theirs
+    // is stored).  Part 0: what U needs (T K~, T, the values); part 1: what O needs (Q~ - M K~, M); part 2: what moves S (K^, decays)
+    constexpr int PF = NBW <= 2 ? 4 : 3, VN = DELTA ? 1 : 4, NW = DELTA ? NBW : 1;
+    f4 rq_[PF][NBW], rk_[PF][NBW], rw_[PF][NW], rd_[PF][ROWS ? NBW : 1];
+    float rm_[PF], rt_[PF];
+    E rv_[PF][VN];
+    uint32_t v_off[VN], v_end[VN];                         // the lane's values within a chunk, and within the last one
+#pragma unroll
+    for (int e = 0; e < VN; ++e) {
+        const int tok = 4 * g + (DELTA ? w : e), col = v_ok ? vcol : vdim - 1;
+        v_off[e] = (uint32_t)((tok * a.ldv + col) * sizeof(E));
+        v_end[e] = (uint32_t)(((tok < n_last ? tok : n_last - 1) * a.ldv + col) * sizeof(E));
+    }
+    auto fetch = [&](int i, int u, int part) {
+        const bool last = i >= n_chunk - 1;
+        i = last ? n_chunk - 1 : i;
         const float* p = rec + i * stride;
+        if (part == 0) {
+            const E* pv = V + (int64_t)(CT * i) * a.ldv;
 #pragma unroll
-        for (int j = 0; j < NBW; ++j) {
-            // (a wave's tiles past the last one repeat it, and their rows of S stay zero)
-            const bool in = w * NBW + j < NT;
-            const int b = in ? w * NBW + j : NT - 1;
-            const f4 zero = f4{0.f, 0.f, 0.f, 0.f};
-            nq[j] = *reinterpret_cast<const f4*>(p + (b * 64 + lane) * 4);
-            const f4 xk = *reinterpret_cast<const f4*>(p + (NT + b) * 256 + lane * 4);
-            nk[j] = in ? xk : zero;
-            if (DELTA) nw[DELTA ? j : 0] = *reinterpret_cast<const f4*>(p + (2 * NT + b) * 256 + lane * 4);
-            nd[j] = *reinterpret_cast<const f4*>(p + NT * 768 + b * 16 + 4 * g);
-        }
-        nm = p[NT * 784 + w * 64 + lane];
-        if (DELTA) nt = p[NT * 784 + 256 + w * 64 + lane];
+            for (int e = 0; e < VN; ++e) rv_[u][e] = at<E>(pv, last ? v_end[e] : v_off[e]);
+            if (DELTA) {
+                rt_[u] = at<float>(p + w_mt + NT * 784 + 256, 4 * lane);
 #pragma unroll
-        for (int e = 0; e < VN; ++e) {
-            const int tok = 16 * i + 4 * g + (DELTA ? w : e);
-            nv[e] = (tok < count && v_ok) ? to_f32(V[(int64_t)tok * a.ldv]) : 0.0f;
+                for (int j = 0; j < NW; ++j) rw_[u][j] = at<f4>(p + (2 * NT + j) * 256, 16 * lane);
+            }
+        } else if (part == 1) {
+            rm_[u] = at<float>(p + w_mt + NT * 784, 4 * lane);
+#pragma unroll
+            for (int j = 0; j < NBW; ++j) rq_[u][j] = at<f4>(p + j * 256, 16 * lane);
+        } else {
+#pragma unroll
+            for (int j = 0; j < NBW; ++j) {
+                rk_[u][j] = at<f4>(p + (NT + j) * 256, 16 * lane);
+                if (ROWS) rd_[u][ROWS ? j : 0] = at<f4>(p + w_dec + NT * 768 + j * 16, 16 * g);
+            }
         }
+        // (the loads stay in order: a wait for one chunk's must not cover the chunks behind it)
+        __builtin_amdgcn_sched_barrier(0);
     };
-    const int n_chunk = (count + CT - 1) / CT;
-    if (n_chunk > 0) fetch(0);
-    for (int i = 0; i < n_chunk; ++i) {
+#pragma unroll
+    for (int u = 0; u < PF; ++u)
+#pragma unroll
+        for (int part = 0; part < 3; ++part) fetch(u, u, part);
+    const uint32_t o_off = (uint32_t)(((4 * g + w) * a.ldo + vcol) * 4);
+    const f4 zero = f4{0.f, 0.f, 0.f, 0.f};
+    // the outputs of chunk i, whose parts the waves left in LDS before the last barrier: wave w writes the tokens 4 g + w
+    auto emit = [&](int i) {
+        const float(&r)[4][64] = red_o[i & 1][w];
+        const float ov = (r[0][lane] + r[1][lane]) + (r[2][lane] + r[3][lane]);
+        float* po = a.out + (row0 + CT * i) * a.ldo + (int64_t)h * vdim;
+        if (CT * i + 4 * g + w < count && v_ok) *reinterpret_cast<float*>(reinterpret_cast<char*>(po) + o_off) = ov;
+    };
+    auto work = [&](int i, int u, bool refill) {           // chunk i out of slot u
         const int buf = i & 1;
-        f4 cq[NBW], ck[NBW], cw[DELTA ? NBW : 1], cd[NBW];
         float cv[VN];
-        const float cm = nm, ct = nt;
 #pragma unroll
-        for (int j = 0; j < NBW; ++j) {
-            cq[j] = nq[j], ck[j] = nk[j], cd[j] = nd[j];
-            if (DELTA) cw[DELTA ? j : 0] = nw[DELTA ? j : 0];
-        }
-#pragma unroll
-        for (int e = 0; e < VN; ++e) cv[e] = nv[e];
-        if (i + 1 < n_chunk) fetch(i + 1);
+        for (int e = 0; e < VN; ++e) cv[e] = to_f32(rv_[u][e]);
         const float v_w = DELTA ? cv[0] : (w == 0 ? cv[0] : w == 1 ? cv[VN > 1 ? 1 : 0] : w == 2 ? cv[VN > 2 ? 2 : 0] : cv[VN > 3 ? 3 : 0]);
-        const f4 zero = f4{0.f, 0.f, 0.f, 0.f};
-        // this wave's part of U and O: four of the tokens' values, and its rows of S
-        f4 u = zero, o = mma4(cm, v_w, zero);
-        if (DELTA) u = mma4(ct, v_w, zero);
+        f4 U;
+        if (DELTA) {
+            // this wave's part of U -- four of the tokens' values and its rows of S -- meets the others' in LDS ...
+            f4 part = mma4(rt_[u], v_w, zero);
+#pragma unroll
+            for (int j = 0; j < NW; ++j)
+#pragma unroll
+                for (int e = 0; e < 4; ++e) part = mma4(rw_[u][j][e], S[j][e], part);
+            red_u[DELTA ? buf : 0][w][lane] = part;
+        }
+        if (refill) fetch(i + PF, u, 0);
+        __syncthreads();                                   // (red_u[buf] was last read two barriers ago, red_o[buf] is written after this one)
+        f4 u4[4];
+        if (DELTA) {
+#pragma unroll
+            for (int x = 0; x < 4; ++x) u4[x] = red_u[DELTA ? buf : 0][x][lane];
+        }
+        // ... while its part of O is under way
+        f4 o = mma4(rm_[u], v_w, zero);
 #pragma unroll
         for (int j = 0; j < NBW; ++j)
 #pragma unroll
-            for (int e = 0; e < 4; ++e) {
-                if (DELTA) u = mma4(cw[DELTA ? j : 0][e], S[j][e], u);
-                o = mma4(cq[j][e], S[j][e], o);
-            }
-        if (DELTA) red_u[DELTA ? buf : 0][w][lane] = u;
-#pragma unroll
-        for (int r = 0; r < 4; ++r) red_o[buf][r][w][lane] = o[r];
-        __syncthreads();                                   // (buffer `buf` was last read two barriers ago)
-        f4 U;
+            for (int e = 0; e < 4; ++e) o = mma4(rq_[u][j][e], S[j][e], o);
+        if (refill) fetch(i + PF, u, 1);
+        if (i > 0) emit(i - 1);
         if (DELTA) {
-            const f4 u0 = red_u[DELTA ? buf : 0][0][lane], u1 = red_u[DELTA ? buf : 0][1][lane], u2 = red_u[DELTA ? buf : 0][2][lane],
-                     u3 = red_u[DELTA ? buf : 0][3][lane];
-#pragma unroll
-            for (int r = 0; r < 4; ++r) U[r] = (u0[r] + u1[r]) + (u2[r] + u3[r]);
+            U = (u4[0] + u4[1]) + (u4[2] + u4[3]);
         } else {
 #pragma unroll
             for (int r = 0; r < 4; ++r) U[r] = cv[DELTA ? 0 : r];
         }
 #pragma unroll
-        for (int j = 0; j < NBW; ++j) {
-            f4 sj = S[j];
+        for (int r = 0; r < 4; ++r) red_o[buf][r][w][lane] = o[r];
+        const float dec = i == n_chunk - 1 ? dec_last : dec_full;
 #pragma unroll
-            for (int r = 0; r < 4; ++r) sj[r] *= cd[j][r];
+        for (int j = 0; j < NBW; ++j)
 #pragma unroll
-            for (int e = 0; e < 4; ++e) sj = mma4(ck[j][e], U[e], sj);
-            S[j] = sj;
-        }
-        // wave w writes the tokens 4 g + w
-        const int tok = 16 * i + 4 * g + w;
-        const float ov = (red_o[buf][w][0][lane] + red_o[buf][w][1][lane]) + (red_o[buf][w][2][lane] + red_o[buf][w][3][lane]);
-        if (tok < count && v_ok) a.out[(row0 + tok) * a.ldo + (int64_t)h * vdim + vcol] = ov;
+            for (int r = 0; r < 4; ++r) S[j][r] *= ROWS ? rd_[u][ROWS ? j : 0][r] : dec;
+#pragma unroll
+        for (int e = 0; e < 4; ++e)
+#pragma unroll
+            for (int j = 0; j < NBW; ++j) S[j] = mma4(rk_[u][j][e], U[e], S[j]);
+        if (refill) fetch(i + PF, u, 2);
+    };
+    // (whole rounds of the ring without a branch between them, then the chunks that are left)
+    int i0 = 0;
+    for (; i0 + PF <= n_chunk; i0 += PF) {
+#pragma unroll
+        for (int u = 0; u < PF; ++u) work(i0 + u, u, true);
     }
+#pragma unroll
+    for (int u = 0; u < PF - 1; ++u)
+        if (i0 + u < n_chunk) work(i0 + u, u, false);
+    __syncthreads();
+    emit(n_chunk - 1);
     if (!v_ok) return;
 #pragma unroll
     for (int i = 0; i < NBW; ++i)
@@ -510,10 +595,17 @@ template <typename E, int NBW>
 void launch_scan(const pcb_rec_args& a, hipStream_t stream) {
     // (heads run fastest: a head's column blocks meet its records in one XCD's L2)
     const dim3 grid(a.H, pcb_ceil_div(a.vdim, 16), a.n_reqs), block(256);
-    if (a.beta)
-        hipLaunchKernelGGL((rec_scan_kernel<E, NBW, true>), grid, block, 0, stream, a);
-    else
-        hipLaunchKernelGGL((rec_scan_kernel<E, NBW, false>), grid, block, 0, stream, a);
+    if (a.beta) {
+        if (a.ld)
+            hipLaunchKernelGGL((rec_scan_kernel<E, NBW, true, true>), grid, block, 0, stream, a);
+        else
+            hipLaunchKernelGGL((rec_scan_kernel<E, NBW, true, false>), grid, block, 0, stream, a);
+    } else {
+        if (a.ld)
+            hipLaunchKernelGGL((rec_scan_kernel<E, NBW, false, true>), grid, block, 0, stream, a);
+        else
+            hipLaunchKernelGGL((rec_scan_kernel<E, NBW, false, false>), grid, block, 0, stream, a);
+    }
 }
 
 template <typename E>
@@ -566,6 +658,7 @@ int check(const pcb_rec_args* a, const char* what) {
                     a->vdim > 0 && a->ldq >= (int64_t)a->Hk * a->dim && a->ldk >= (int64_t)a->Hk * a->dim && a->ldv >= (int64_t)a->H * a->vdim &&
                     a->slot_stride >= (int64_t)a->H * a->dim * a->vdim,
                 PCB_ERR_ARG, "%s: bad sizes (up to 256 key columns per head)", what);
+    PCB_REQUIRE(a->ldv < (1 << 26) && a->ldo < (1 << 24), PCB_ERR_ARG, "%s: rows too long", what);
     PCB_REQUIRE(a->rot_dims >= 0 && a->rot_dims % 2 == 0 && a->rot_dims <= a->dim && (a->rot_dims == 0 || a->rot || a->n_reqs == 0), PCB_ERR_ARG,
                 "%s: rotated columns come in pairs inside the head, with their table of cosines and sines", what);
     PCB_REQUIRE(a->n_reqs == 0 || ((a->decay != nullptr) != (a->ld != nullptr)), PCB_ERR_ARG,
@@ -577,7 +670,7 @@ int check(const pcb_rec_args* a, const char* what) {
 }  // namespace
 
 PCB_EXPORT int64_t pcb_rec_scratch(int32_t n_chunks, int32_t H, int32_t dim) {
-    return n_chunks > 0 && H > 0 && dim > 0 && dim <= 256 ? (int64_t)n_chunks * H * rec_record(dim) : 0;
+    return n_chunks > 0 && H > 0 && dim > 0 && dim <= 256 ? (int64_t)n_chunks * H * rec_record(rec_columns(dim) / 16) : 0;
 }
 
 PCB_EXPORT int pcb_rec_prompt(const pcb_rec_args* a, void* stream) {

@@ -256,19 +256,17 @@ __global__ __launch_bounds__(256) void conv_step_kernel(const E* __restrict__ x,
     const E* wc = w + (int64_t)ch * taps;
     const int m1 = taps - 1;
     const E xv = x[r * ldx + ch];
-    E old[MAX_TAPS];
+    float old[MAX_TAPS];
 #pragma unroll
-    for (int m = 0; m < MAX_TAPS; ++m) {
-        if (m >= m1) break;
-        old[m] = pos - m1 + m >= 0 ? st[(int64_t)m * C] : from_f32<E>(0.0f);      // (state row m: the token m1 - m before this one)
-    }
+    for (int m = 0; m < MAX_TAPS; ++m)                     // (state row m: the token m1 - m before this one)
+        old[m] = m < m1 && pos - m1 + m >= 0 ? to_f32(st[(int64_t)m * C]) : 0.0f;
     float acc = bias ? to_f32(bias[ch]) : 0.0f;
 #pragma unroll
-    for (int m = 0; m < MAX_TAPS; ++m) {
-        if (m >= m1) break;
-        acc += to_f32(wc[m]) * to_f32(old[m]);
-        if (m > 0) st[(int64_t)(m - 1) * C] = old[m];
-    }
+    for (int m = 0; m < MAX_TAPS; ++m)
+        if (m < m1) {
+            acc += to_f32(wc[m]) * old[m];
+            if (m > 0) st[(int64_t)(m - 1) * C] = from_f32<E>(old[m]);
+        }
     acc += to_f32(wc[m1]) * to_f32(xv);
     if (m1 > 0) st[(int64_t)(m1 - 1) * C] = xv;
     if (silu) acc = acc / (1.0f + expf(-acc));
@@ -303,24 +301,20 @@ __global__ __launch_bounds__(256) void conv_state_kernel(const E* __restrict__ x
     const int ch = blockIdx.y * 256 + threadIdx.x;
     if (ch >= C) return;
     E* st = state + (int64_t)slot * slot_stride;
-    E keep[MAX_TAPS];
+    float keep[MAX_TAPS];
     const int m1 = taps - 1;
 #pragma unroll
     for (int m = 0; m < MAX_TAPS; ++m) {
-        if (m >= m1) break;
         const int p = pos0 + count - m1 + m;              // the position state row m holds after the step
-        E v = from_f32<E>(0.0f);
-        if (p >= pos0)
-            v = x[(int64_t)(row0 + p - pos0) * ldx + ch];
-        else if (p >= 0)
-            v = st[(int64_t)(m + count) * C + ch];
-        keep[m] = v;
+        keep[m] = 0.0f;
+        if (m < m1 && p >= pos0)
+            keep[m] = to_f32(x[(int64_t)(row0 + p - pos0) * ldx + ch]);
+        else if (m < m1 && p >= 0)
+            keep[m] = to_f32(st[(int64_t)(m + count) * C + ch]);
     }
 #pragma unroll
-    for (int m = 0; m < MAX_TAPS; ++m) {
-        if (m >= m1) break;
-        st[(int64_t)m * C + ch] = keep[m];
-    }
+    for (int m = 0; m < MAX_TAPS; ++m)
+        if (m < m1) st[(int64_t)m * C + ch] = from_f32<E>(keep[m]);
 }
 
 // ---- selective scan ---------------------------------------------------------------------------------------------------------------
