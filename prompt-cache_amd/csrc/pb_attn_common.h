@@ -42,12 +42,6 @@ __device__ __forceinline__ f4 mma_p(const Frag<bf16_t>& v, const PFrag<bf16_t>& 
 }
 __device__ __forceinline__ f4 mma_p(const Frag<float>& v, const PFrag<float>& p, f4 c) { return mma(v, p.hi, c); }
 
-// four numbers as neighbouring elements of E (p aligned to the four)
-__device__ __forceinline__ void store4(bf16_t* p, float a, float b, float c, float d) {
-    *reinterpret_cast<uint2*>(p) = uint2{(uint32_t)bf16_bits(a) | ((uint32_t)bf16_bits(b) << 16), (uint32_t)bf16_bits(c) | ((uint32_t)bf16_bits(d) << 16)};
-}
-__device__ __forceinline__ void store4(float* p, float a, float b, float c, float d) { *reinterpret_cast<float4*>(p) = float4{a, b, c, d}; }
-
 // ---- value operands out of an LDS tile kept key by key ([key][column], ld elements per key) ------------------------------------------
 // The second product is O^T = V^T P^T: its A operand wants, per lane (value column l & 15, group l >> 4), eight keys of that column.  Key
 // k index (group g, e) stands for key 4 g + e (e < 4) and 16 + 4 g + e - 4 (e >= 4) of the 32-key step -- what the lanes hold of the

@@ -164,6 +164,11 @@ __device__ __forceinline__ void load4(const float* p, bool vec, int valid, float
         for (int i = 0; i < 4; ++i) o[i] = i < valid ? p[i] : 0.0f;
     }
 }
+// four numbers as neighbouring elements of E (p aligned to the four)
+__device__ __forceinline__ void store4(bf16_t* p, float a, float b, float c, float d) {
+    *reinterpret_cast<uint2*>(p) = uint2{(uint32_t)bf16_bits(a) | ((uint32_t)bf16_bits(b) << 16), (uint32_t)bf16_bits(c) | ((uint32_t)bf16_bits(d) << 16)};
+}
+__device__ __forceinline__ void store4(float* p, float a, float b, float c, float d) { *reinterpret_cast<float4*>(p) = float4{a, b, c, d}; }
 
 // result tile: lane l holds column (l & 15), rows 4 * (l >> 4) + r, r = 0..3
 

@@ -3,6 +3,8 @@
 // mixture of experts (bucketing pairs by expert, summing the pairs' results back into the stream).  All reductions fp32.
 #include <string.h>
 
+#include <type_traits>
+
 #include "pb_common.h"
 
 static thread_local char g_err[512] = "";
@@ -429,6 +431,49 @@ __global__ __launch_bounds__(256) void gated_group_norm_kernel(const float* __re
     }
 }
 
+// the same for heads of up to 4 LPG columns, read and written four columns at a time: LPG lanes share a (row, head) pair, each column is
+// read once and waits in registers for the sum
+template <typename E, int LPG>
+__global__ __launch_bounds__(256) void gated_head_norm_kernel(const float* __restrict__ x, int64_t ldx, const float* __restrict__ gain,
+                                                              const E* __restrict__ gate, int64_t ldg, E* __restrict__ out, int64_t ldo,
+                                                              float eps, int per, int group, int64_t n_pairs) {
+    const int64_t pair = (int64_t)blockIdx.x * (256 / LPG) + threadIdx.x / LPG;
+    if (pair >= n_pairs) return;                            // (whole groups of lanes leave: the sums below stay inside a group)
+    const int64_t r = pair / per;
+    const int c0 = (int)(pair % per) * group, c = threadIdx.x % LPG * 4;
+    const bool ok = c < group;
+    float v[4] = {0.0f, 0.0f, 0.0f, 0.0f}, gt[4] = {1.0f, 1.0f, 1.0f, 1.0f};
+    if (ok) load4(x + r * ldx + c0 + c, true, 4, v);
+    if (ok && gate) load4(gate + r * ldg + c0 + c, true, 4, gt);
+    float ss = v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3];
+#pragma unroll
+    for (int o = LPG / 2; o > 0; o >>= 1) ss += __shfl_xor(ss, o, 64);
+    const float inv = 1.0f / sqrtf(ss / (float)group + eps);
+    if (!ok) return;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) v[e] *= inv * (gain ? gain[c0 + c + e] : 1.0f) * gt[e];
+    store4(out + r * ldo + c0 + c, v[0], v[1], v[2], v[3]);
+}
+
+template <typename E>
+bool launch_head_norm(const float* x, int64_t ldx, const float* gain, const void* gate, int64_t ldg, void* out, int64_t ldo, float eps, int n_rows,
+                      int cols, int group, hipStream_t stream) {
+    constexpr uintptr_t A4 = 4 * sizeof(E);
+    if (group > 256 || group % 4 || ldx % 4 || ldo % 4 || (gate && ldg % 4) || (uintptr_t)x % 16 || (uintptr_t)out % A4 || (uintptr_t)gate % A4) return false;
+    const int per = cols / group;
+    const int64_t pairs = (int64_t)n_rows * per;
+    auto go = [&](auto l) {
+        constexpr int LPG = decltype(l)::value;
+        hipLaunchKernelGGL((gated_head_norm_kernel<E, LPG>), dim3((unsigned)((pairs * LPG + 255) / 256)), dim3(256), 0, stream, x, ldx, gain, (const E*)gate,
+                           ldg, (E*)out, ldo, eps, per, group, pairs);
+        return true;
+    };
+    if (group <= 32) return go(std::integral_constant<int, 8>{});
+    if (group <= 64) return go(std::integral_constant<int, 16>{});
+    if (group <= 128) return go(std::integral_constant<int, 32>{});
+    return go(std::integral_constant<int, 64>{});
+}
+
 // one workgroup per row; the row waits in LDS between the two sums (width * 4 bytes of dynamic LDS)
 template <typename E>
 __global__ __launch_bounds__(1024) void post_norm_kernel(pcb_post_norm_args a) {
@@ -656,7 +701,12 @@ PCB_EXPORT int pcb_gated_norm(const float* x, int64_t ldx, const float* gain, co
     if (n_rows == 0) return PCB_OK;
     PCB_REQUIRE(x && out, PCB_ERR_ARG, "pcb_gated_norm: null pointer");
     if (gate_first || skip) group_cols = group_cols > 0 ? group_cols : cols;       // (the per-group kernel knows these two)
-    if ((group_cols > 0 && group_cols < cols) || gate_first || skip) {
+    // (groups are normed with or without a gain, a whole row by the kernel below only with one)
+    if ((group_cols > 0 && (group_cols < cols || !gain)) || gate_first || skip) {
+        if (!gate_first && !skip &&
+            (dtype == PCB_BF16 ? launch_head_norm<bf16_t>(x, ldx, gain, gate, ldg, out, ldo, eps, n_rows, cols, group_cols, (hipStream_t)stream)
+                               : launch_head_norm<float>(x, ldx, gain, gate, ldg, out, ldo, eps, n_rows, cols, group_cols, (hipStream_t)stream)))
+            return pcb_check_launch("gated_head_norm_kernel");
         const int64_t pairs = (int64_t)n_rows * (cols / group_cols);
         const bool wide = group_cols >= 512;
         const dim3 grid((unsigned)(wide ? pairs : (pairs + 3) / 4));
