@@ -715,7 +715,7 @@ def run_dibizen(args):
     `mamba1` = four layers of that mixer alone, which is what prices each mixer's kernels.  Random weights, synthetic tokens."""
     import torch
     import __graft_entry__ as ge
-    ge.build()
+    ge.ensure_built()
     from promptcache_amd.model import Dibizen, Kazolorn
     from promptcache_amd.model.config import DibizenShape, KazolornShape
     dev = "cuda:0"
@@ -756,7 +756,7 @@ def run_fivesun(args):
     positions, latent attention a window of 1024 over a latent of 192 + 64 columns.  Random weights, synthetic tokens."""
     import torch
     import __graft_entry__ as ge
-    ge.build()
+    ge.ensure_built()
     from promptcache_amd.model import Dibizen, Fivesun
     from promptcache_amd.model.config import DibizenShape, FivesunShape
     dev = "cuda:0"
@@ -797,7 +797,7 @@ def run_bepepel(args):
     with 128 states.  Random weights, synthetic tokens."""
     import torch
     import __graft_entry__ as ge
-    ge.build()
+    ge.ensure_built()
     from promptcache_amd.model import Bepepel, Dibizen
     from promptcache_amd.model.config import BepepelShape, DibizenShape
     dev = "cuda:0"
@@ -835,7 +835,7 @@ def run_pikadra(args):
     weights, synthetic tokens."""
     import torch
     import __graft_entry__ as ge
-    ge.build()
+    ge.ensure_built()
     from promptcache_amd.model import Fivesun, Pikadra
     from promptcache_amd.model.config import FivesunShape, PikadraShape
     dev = "cuda:0"
@@ -875,7 +875,7 @@ def run_venitar(args):
     the middle two layers run twice (six layer runs).  The window and the blocks have 1024 positions.  Random weights, synthetic tokens."""
     import torch
     import __graft_entry__ as ge
-    ge.build()
+    ge.ensure_built()
     from promptcache_amd.model import Bepepel, Fivesun, Venitar
     from promptcache_amd.model.config import BepepelShape, FivesunShape, VenitarShape
     dev = "cuda:0"
@@ -916,7 +916,7 @@ def run_kazolorn(args):
     Random weights, synthetic tokens, 4 layers (throughput per layer is what is compared)."""
     import torch
     import __graft_entry__ as ge
-    ge.build()
+    ge.ensure_built()
     from promptcache_amd import BatchEngine
     from promptcache_amd.model import Kazolorn, Mpt
     from promptcache_amd.model.config import KazolornShape, MptShape
@@ -1089,7 +1089,7 @@ def main():
 
     import __graft_entry__ as ge
     if rank == 0:
-        ge.build()
+        ge.ensure_built()
     barrier()
     from promptcache_amd import CacheEngine, Prompt, synth
     from promptcache_amd.model import Llama2

@@ -352,9 +352,12 @@ __global__ __launch_bounds__(256) void rec_scan_kernel(pcb_rec_args a) {
     const uint32_t o_off = (uint32_t)(((4 * g + w) * a.ldo + vcol) * 4);
     const f4 zero = f4{0.f, 0.f, 0.f, 0.f};
     // the outputs of chunk i, whose parts the waves left in LDS before the last barrier: wave w writes the tokens 4 g + w
-    auto emit = [&](int i) {
-        const float(&r)[4][64] = red_o[i & 1][w];
-        const float ov = (r[0][lane] + r[1][lane]) + (r[2][lane] + r[3][lane]);
+    auto parts_of = [&](int i, float (&r)[4]) {
+#pragma unroll
+        for (int x = 0; x < 4; ++x) r[x] = red_o[i & 1][w][x][lane];
+    };
+    auto emit = [&](int i, const float (&r)[4]) {
+        const float ov = (r[0] + r[1]) + (r[2] + r[3]);
         float* po = a.out + (row0 + CT * i) * a.ldo + (int64_t)h * vdim;
         if (CT * i + 4 * g + w < count && v_ok) *reinterpret_cast<float*>(reinterpret_cast<char*>(po) + o_off) = ov;
     };
@@ -374,9 +377,10 @@ __global__ __launch_bounds__(256) void rec_scan_kernel(pcb_rec_args a) {
                 for (int e = 0; e < 4; ++e) part = mma4(rw_[u][j][e], S[j][e], part);
             red_u[DELTA ? buf : 0][w][lane] = part;
         }
-        if (refill) fetch(i + PF, u, 0);
         __syncthreads();                                   // (red_u[buf] was last read two barriers ago, red_o[buf] is written after this one)
         f4 u4[4];
+        float before[4];                                   // (of the chunk before; the first chunk's are not used)
+        parts_of(i - 1, before);
         if (DELTA) {
 #pragma unroll
             for (int x = 0; x < 4; ++x) u4[x] = red_u[DELTA ? buf : 0][x][lane];
@@ -386,9 +390,12 @@ __global__ __launch_bounds__(256) void rec_scan_kernel(pcb_rec_args a) {
 #pragma unroll
         for (int j = 0; j < NBW; ++j)
 #pragma unroll
-            for (int e = 0; e < 4; ++e) o = mma4(rq_[u][j][e], S[j][e], o);
+            for (int e = 0; e < 4; ++e) {
+                o = mma4(rq_[u][j][e], S[j][e], o);
+                if (refill && j == 0 && e == 3) fetch(i + PF, u, 0);       // (loads go out between products: a wave's queue of them is short)
+            }
         if (refill) fetch(i + PF, u, 1);
-        if (i > 0) emit(i - 1);
+        if (i > 0) emit(i - 1, before);
         if (DELTA) {
             U = (u4[0] + u4[1]) + (u4[2] + u4[3]);
         } else {
@@ -418,7 +425,9 @@ __global__ __launch_bounds__(256) void rec_scan_kernel(pcb_rec_args a) {
     for (int u = 0; u < PF - 1; ++u)
         if (i0 + u < n_chunk) work(i0 + u, u, false);
     __syncthreads();
-    emit(n_chunk - 1);
+    float before[4];
+    parts_of(n_chunk - 1, before);
+    emit(n_chunk - 1, before);
     if (!v_ok) return;
 #pragma unroll
     for (int i = 0; i < NBW; ++i)

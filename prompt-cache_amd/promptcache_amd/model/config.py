@@ -1143,7 +1143,7 @@ class VenitarShape:
         def attention(a, mask_as):
             heads, dim = int(a["heads"]), int(a["dim"])
             return VenitarAttention(heads=heads, kv_heads=int(a.get("kv_heads") or heads), dim=dim, vdim=int(a.get("vdim") or dim),
-                                    scale=float(a["scale"]), rot=VenitarRot.from_config(a.get("rot")),
+                                    scale=float(a.get("scale", dim ** -0.5)), rot=VenitarRot.from_config(a.get("rot")),
                                     **{mask_as: int((a.get("mask") or {}).get("size") or 0)})
 
         layers = []
@@ -1158,8 +1158,8 @@ class VenitarShape:
             elif kind == "parallel":
                 b = m["right"]
                 heads, dim = int(b["heads"]), int(b["dim"])
-                lay = VenitarLayer(kind, left=attention(m["left"], "window"), left_scale=float(m["left_scale"]),
-                                   right_scale=float(m["right_scale"]),
+                lay = VenitarLayer(kind, left=attention(m["left"], "window"), left_scale=float(m.get("left_scale", 1.0)),
+                                   right_scale=float(m.get("right_scale", 1.0)),
                                    right=VenitarDelta(heads=heads, kv_heads=int(b.get("kv_heads") or heads), dim=dim,
                                                       vdim=int(b.get("vdim") or dim), conv=int(b["conv"])))
             else:
@@ -1173,7 +1173,7 @@ class VenitarShape:
                     raise ValueError(f"layer {i}: a feed-forward of width {lay.ff}")
             layers.append(lay)
         loop = c.get("loop") or {}
-        shape = cls(vocab_size=int(c["vocab"]), hidden_size=int(c["width"]), norm_eps=float(c["norm"]["eps"]), layers=layers,
+        shape = cls(vocab_size=int(c["vocab"]), hidden_size=int(c["width"]), norm_eps=float((c.get("norm") or {}).get("eps", 1e-6)), layers=layers,
                     embed_scale=float((c.get("embedding") or {}).get("scale", 1.0)), loop_start=int(loop.get("start", 0)),
                     loop_stop=int(loop.get("stop", len(layers))) if loop else 0, loop_times=int(loop.get("times", 1)) if loop else 0, name=name)
         shape.check()
